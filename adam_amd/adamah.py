@@ -36,6 +36,9 @@ DECODE_RUNTIME_SEQ_LEN = 0xFFFFFFFD
  DECODE_OP_ROW_COPY_OFFSET, DECODE_OP_ATTN_SOFTMAX_VALUE) = range(10, 26)
 (DECODE_OP_FUSED_QKV_T_XQ4, DECODE_OP_FUSED_GATEUP_T_XQ4, DECODE_OP_FUSED_QKV_T_XQ8, DECODE_OP_FUSED_GATEUP_T_XQ8,
  DECODE_OP_FUSED_GATEUP_ACT_T_XQ8) = range(26, 31)
+# layered mixers over bfloat16 weights (no counterpart in the reference)
+(DECODE_OP_LINEAR, DECODE_OP_LINEAR_ARGMAX, DECODE_OP_MERGE_NORM, DECODE_OP_DELTA_RULE, DECODE_OP_RETENTION,
+ DECODE_OP_CHUNK_ATTENTION) = range(31, 37)
 
 (OP_NEG, OP_ABS, OP_SQRT, OP_EXP, OP_LOG, OP_TANH, OP_RELU, OP_GELU, OP_SIN, OP_COS, OP_TAN, OP_ASIN,
  OP_ACOS, OP_ATAN, OP_SINH, OP_COSH, OP_SIGMOID, OP_SWISH, OP_MISH, OP_SELU, OP_ELU, OP_LEAKY_RELU,
@@ -54,6 +57,26 @@ class DecodePlanOp(ctypes.Structure):
     """Flat decode-plan record: 16 x u32 + 2 x f32 (reference adamah.c:175-194)."""
     _fields_ = [(n, u32) for n in ("kind", "map_id", "map_id2", "op_code", "h0", "h1", "h2", "h3", "h4",
                                    "h5", "u0", "u1", "u2", "u3", "u4", "u5")] + [("f0", f32c), ("f1", f32c)]
+
+
+def _spec(name, fields, floats=()):
+    """A struct of 32-bit words that travels in an uploaded handle (include/adamah_hip.h names the fields)."""
+    return type(name, (ctypes.Structure,), {
+        "_fields_": [(n, f32c if n in floats else u32) for n in fields.split()],
+        "words": lambda self: np.frombuffer(bytes(self), np.uint32).copy()})
+
+
+LinearSpec = _spec("LinearSpec", "w n k k_stride src src_stride groups eps wt wt_len gate gate_stride gate_act opnd ready out "
+                   "out_stride epi out_opnd out_opnd_stride", ("eps",))
+MergeSpec = _spec("MergeSpec", "a b stride wa wb dst dst_stride dim eps scale", ("eps", "scale"))
+DeltaSpec = _spec("DeltaSpec", "heads kv_heads dim vdim taps x x_stride x_b cq ck cv a_log dt_bias out out_stride state_map s_off "
+                  "conv_off seq_stride")
+RetentionSpec = _spec("RetentionSpec", "heads dim vdim rot_dims freq decay x x_stride x_q x_k x_v out out_stride state_map s_off "
+                      "seq_stride")
+ChunkAttnSpec = _spec("ChunkAttnSpec", "heads kv_heads dim vdim chunk x x_stride x_q x_k x_v r1 r2 scale eps out out_stride "
+                      "cache_map k_off v_off seq_stride", ("scale", "eps"))
+GATE_NONE, GATE_SIGMOID, GATE_SILU = 0, 1, 2
+EPI_STORE, EPI_ADD, EPI_SWIGLU = 0, 1, 2
 
 
 def _resolve_lib_path(lib_path=None):
@@ -134,6 +157,9 @@ _SIGS = {
     "map_fused_qkv_t_xq4_dev": (i32, [_U] * 13), "map_fused_qkv_t_xq8_dev": (i32, [_U] * 13),
     "map_fused_gateup_t_xq4_dev": (i32, [_U] * 10), "map_fused_gateup_t_xq8_dev": (i32, [_U] * 10),
     "map_fused_gateup_act_t_xq8_dev": (i32, [_U] * 8),
+    "adamah_linear_dev": (i32, [_U] * 6), "adamah_linear_argmax_dev": (i32, [_U] * 6), "adamah_merge_norm_dev": (i32, [_U] * 3),
+    "adamah_delta_rule_dev": (i32, [_U] * 10), "adamah_retention_dev": (i32, [_U] * 6),
+    "adamah_chunk_attention_dev": (i32, [_U] * 6),
     # timing helpers for benchmarks (HIP events on the library's own stream)
     "adamah_hip_timer_begin": (i32, []), "adamah_hip_timer_end": (f32c, []),
     "adamah_hip_debug_dequant": (i32, [_U, u64, u64, pf32]),
@@ -706,6 +732,26 @@ class Adamah:
         ret = self._lib.adamah_decode_step(plan_id, pos, seq_len)
         if ret != 0:
             raise RuntimeError(f"adamah_decode_step failed with code {ret}")
+
+    # ---- layered mixers over bfloat16 weights (include/adamah_hip.h; argument order as there) ----------
+    def linear_dev(self, map_act, map_opnd, map_wt, spec_handle, rows_handle, rows):
+        self._op("adamah_linear_dev", map_act, map_opnd, map_wt, spec_handle, rows_handle, rows)
+
+    def linear_argmax_dev(self, map_act, map_opnd, map_wt, spec_handle, dst_handle, rows):
+        self._op("adamah_linear_argmax_dev", map_act, map_opnd, map_wt, spec_handle, dst_handle, rows)
+
+    def merge_norm_dev(self, map_act, spec_handle, rows):
+        self._op("adamah_merge_norm_dev", map_act, spec_handle, rows)
+
+    def delta_rule_dev(self, map_act, map_opnd, map_wt, spec_handle, decay_handle, gate_handle, n_seq, rows, seq0, pos):
+        self._op("adamah_delta_rule_dev", map_act, map_opnd, map_wt, spec_handle, decay_handle, gate_handle, n_seq, rows,
+                 seq0, pos)
+
+    def retention_dev(self, map_act, spec_handle, n_seq, rows, seq0, pos):
+        self._op("adamah_retention_dev", map_act, spec_handle, n_seq, rows, seq0, pos)
+
+    def chunk_attention_dev(self, map_act, spec_handle, n_seq, rows, seq0, pos):
+        self._op("adamah_chunk_attention_dev", map_act, spec_handle, n_seq, rows, seq0, pos)
 
     # ---- benchmark / test helpers (not part of the reference surface) ------------------
     def timer_begin(self):

@@ -7,7 +7,7 @@ from concurrent.futures import ThreadPoolExecutor
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 OUT = os.path.join(HERE, "libadamah_hip.so")
-SOURCES = ["runtime.hip", "gemv_q.hip", "gemv_mfma.hip", "gemm_q4_mfma.hip", "fuse.hip", "norm_rope.hip", "rowprep.hip", "attention.hip", "attn_decode.hip", "attn_prefill.hip", "elementwise.hip", "sampling.hip", "topk_fused.hip", "fused_proj.hip", "token_feed.hip", "probe.hip"]
+SOURCES = ["runtime.hip", "gemv_q.hip", "gemv_mfma.hip", "gemm_q4_mfma.hip", "fuse.hip", "norm_rope.hip", "rowprep.hip", "attention.hip", "attn_decode.hip", "attn_prefill.hip", "elementwise.hip", "sampling.hip", "topk_fused.hip", "fused_proj.hip", "token_feed.hip", "linear_bf16.hip", "recurrent.hip", "attn_chunk.hip", "probe.hip"]
 # -amdgpu-kernarg-preload-count: the first 14 dwords of a kernel's arguments (whole scalars / pointers, in order) are
 # in SGPRs when a wave starts instead of being fetched from the argument block -- one trip to memory less before a
 # kernel's first loads (Q4 GEMV 5.8 -> 5.4 us at 4096x4096).  The hot kernels order their arguments for it.
@@ -53,7 +53,9 @@ def build(verbose=True, jobs=None):
         for s, out in zip(SOURCES, ex.map(one, range(len(SOURCES)))):
             if verbose and out.strip():
                 print(f"[{s}]\n{out}")
-    _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-fno-gpu-rdc", *objs, "-o", OUT])
+    part = f"{OUT}.{os.getpid()}"
+    _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-fno-gpu-rdc", *objs, "-o", part])
+    os.replace(part, OUT)          # a library that is there is whole
     if verbose:
         print(f"built {OUT} ({os.path.getsize(OUT) // 1024} KiB)")
     return OUT

@@ -46,7 +46,7 @@ struct Map {
   bool active = false;
   uint32_t dtype = 0, word_size = 0, pack_size = 0, n_packs = 0, group_size = 0;
   uint64_t n_elems = 0, total_bytes = 0, n_groups = 0;
-  uint8_t* buf = nullptr;   // f32 values, or packed codes (Q4: 2 per byte, Q8: 1 per byte)
+  uint8_t* buf = nullptr;   // f32 or bf16 values, or packed codes (Q4: 2 per byte, Q8: 1 per byte)
   float2* qp = nullptr;     // (scale, zp) per group
   __half* d16 = nullptr;    // fp16 scale per group, valid for groups [0, block16_groups)
   uint64_t block16_groups = 0;
@@ -201,6 +201,9 @@ int launch_attn_combine_dev(Map* m, const float* partial, const uint32_t* lo_dev
                             uint32_t n_splits);
 void attn_decode_release();
 void attn_prefill_release();   // attn_prefill.hip: the transposed V tiles (shutdown)
+void linear_release();          // linear_bf16.hip, recurrent.hip, attn_chunk.hip: their scratch (shutdown)
+void recurrent_release();
+void attn_chunk_release();
 void token_feed_release();      // frees the pinned ring tokens reach the host through (shutdown)
 
 inline void layout_changed() { g.layout_gen++; }

@@ -407,6 +407,9 @@ void adamah_shutdown(void) { ADAMAH_API();
   attn_decode_release();
   attn_prefill_release();
   token_feed_release();
+  linear_release();
+  recurrent_release();
+  attn_chunk_release();
   g.pend.clear();
   for (int i = 0; i < MAX_PLANS; i++) { g.plans[i].clear(); g.plan_active[i] = false; plan_graph_reset(i); }
   hipStreamDestroy(g.stream);
@@ -480,7 +483,7 @@ uint32_t adamah_get_last_barrier_count(void) { ADAMAH_API(); return g.stats.last
 // ---- maps ------------------------------------------------------------------------------------------
 int adamah_set_dtype(uint32_t dtype) {
   if (!g.initialized || dtype >= DTYPE_COUNT) return ADAMAH_ERR_INVALID;
-  if (dtype == DTYPE_BF16 || dtype == DTYPE_Q6) return ADAMAH_ERR_INVALID;  // storage types not built
+  if (dtype == DTYPE_Q6) return ADAMAH_ERR_INVALID;  // storage type not built
   g.active_dtype = dtype;
   return ADAMAH_OK;
 }
@@ -488,7 +491,7 @@ uint32_t adamah_get_dtype(void) { return g.active_dtype; }
 
 int map_init_dtype(uint32_t id, uint32_t dtype, uint32_t pack_size, uint32_t n_packs, uint32_t group_size) { ADAMAH_API();
   if (!g.initialized || id >= MAX_MAPS || dtype >= DTYPE_COUNT) return ADAMAH_ERR_INVALID;
-  if (dtype == DTYPE_BF16 || dtype == DTYPE_Q6) return ADAMAH_ERR_INVALID;
+  if (dtype == DTYPE_Q6) return ADAMAH_ERR_INVALID;
   Map* m = &g.maps[id];
   g.mem_gen++;   // the fills below rewrite device memory without counting as launches
   layout_changed();
@@ -496,9 +499,9 @@ int map_init_dtype(uint32_t id, uint32_t dtype, uint32_t pack_size, uint32_t n_p
   bool quant = dtype == DTYPE_Q8 || dtype == DTYPE_Q4;
   m->dtype = dtype; m->pack_size = pack_size; m->n_packs = n_packs;
   m->group_size = quant ? group_size : 0;
-  m->word_size = dtype == DTYPE_F32 ? 4 : 1;
+  m->word_size = dtype == DTYPE_F32 ? 4 : dtype == DTYPE_BF16 ? 2 : 1;
   m->n_elems = (uint64_t)pack_size * n_packs;
-  if (dtype == DTYPE_F32) m->total_bytes = m->n_elems * 4;
+  if (dtype == DTYPE_F32 || dtype == DTYPE_BF16) m->total_bytes = m->n_elems * m->word_size;
   else if (dtype == DTYPE_Q8) m->total_bytes = ((m->n_elems + 3) / 4) * 4;
   else m->total_bytes = ((m->n_elems + 7) / 8) * 4;
   size_t alloc = std::max<uint64_t>(m->total_bytes, 4) + 256;   // tail pad keeps 16-byte row loads in bounds
@@ -624,6 +627,7 @@ static int scatter_impl(Map* m, const uint32_t* locs, uint64_t start_pack, bool 
     }
     return check_launch();
   }
+  if (m->dtype == DTYPE_BF16) return ADAMAH_ERR_INVALID;   // 16-bit maps take contiguous ranges only
   uint8_t* src = (uint8_t*)tmp_dev(0, n_vals * es);
   uint32_t* dl = (uint32_t*)tmp_dev(1, (size_t)n_locs * 4);
   if (!src || !dl) return ADAMAH_ERR_MEMORY;
@@ -685,6 +689,7 @@ uint64_t map_gather(uint32_t map_id, const uint32_t* locs, void* data, uint32_t 
   uint32_t start = 0;
   if (locs_contiguous(locs, n_locs, m->n_packs, &start) && (start + (uint64_t)n_locs) * pack_bytes <= m->total_bytes)
     return (uint64_t)(int64_t)d2h(data, m->buf + (size_t)start * pack_bytes, (size_t)n_locs * pack_bytes);
+  if (m->dtype == DTYPE_BF16) return (uint64_t)(int64_t)ADAMAH_ERR_INVALID;
   uint32_t* dl = (uint32_t*)tmp_dev(1, (size_t)n_locs * 4);
   uint8_t* dst = (uint8_t*)tmp_dev(0, (size_t)n_locs * pack_bytes);
   if (!dl || !dst) return (uint64_t)(int64_t)ADAMAH_ERR_MEMORY;
@@ -847,6 +852,13 @@ static int replay_plan(uint32_t plan_id, uint32_t pos, uint32_t seq_len) {
       case 28: ret = map_fused_qkv_t_xq8_dev(op.map_id, op.map_id2, op.h0, op.h1, op.h2, op.h3, op.h4, op.h5, u0, u1, u2, u3, u4); break;
       case 29: ret = map_fused_gateup_t_xq8_dev(op.map_id, op.map_id2, op.h0, op.h1, op.h2, op.h3, op.h4, u0, u1, u2); break;
       case 30: ret = map_fused_gateup_act_t_xq8_dev(op.map_id, op.map_id2, op.h0, op.h1, op.h2, op.h3, u0, u1); break;
+      // layered mixers: rows / sequences travel as the op recorded them, the position is the runtime one
+      case 31: ret = adamah_linear_dev(op.map_id, op.op_code, op.map_id2, op.h0, op.h1, u0); break;
+      case 32: ret = adamah_linear_argmax_dev(op.map_id, op.op_code, op.map_id2, op.h0, op.h1, u0); break;
+      case 33: ret = adamah_merge_norm_dev(op.map_id, op.h0, u0); break;
+      case 34: ret = adamah_delta_rule_dev(op.map_id, op.op_code, op.map_id2, op.h0, op.h1, op.h2, u0, u1, u2, u3); break;
+      case 35: ret = adamah_retention_dev(op.map_id, op.h0, u0, u1, u2, u3); break;
+      case 36: ret = adamah_chunk_attention_dev(op.map_id, op.h0, u0, u1, u2, u3); break;
       default: ret = ADAMAH_ERR_INVALID; break;
     }
     if (ret != ADAMAH_OK) break;

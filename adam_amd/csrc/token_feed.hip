@@ -28,7 +28,7 @@ static uint32_t g_ticket = 0;             // last ticket handed out: 1, 2, ... (
 // out[dst0 + r * E + e] = table[row0 + tok_r * E + e] * scale for the m tokens tok_r = act[token slot r].  Quantised
 // tables are decoded as the dequantising gather does (float(code) * scale_g + zp_g, shaders/src/q4/map_gather.comp).
 // A token outside [0, V) gives a row of zeros, as a gather outside the map does.  tok_by_val: slot r is tok0 + r.
-template <int FMT>   // 0 = float32, 1 = Q4 (two codes a byte), 2 = Q8
+template <int FMT>   // 0 = float32, 1 = Q4 (two codes a byte), 2 = Q8, 3 = bfloat16
 __global__ void __launch_bounds__(256)
 k_embed_tokens(float* act, uint64_t act_elems, const uint8_t* __restrict__ src, uint64_t src_elems, uint64_t row0,
                uint32_t E, uint32_t V, uint32_t total, uint32_t dst0, uint32_t tok0, uint32_t tok_by_val, float scale,
@@ -57,6 +57,7 @@ k_embed_tokens(float* act, uint64_t act_elems, const uint8_t* __restrict__ src, 
   float v = 0.0f;
   if (ok) {
     if (FMT == 0) v = ((const float*)src)[idx];
+    else if (FMT == 3) v = __uint_as_float((uint32_t)((const uint16_t*)src)[idx] << 16);
     else {
       const uint32_t code = FMT == 1 ? ((src[idx >> 1] >> ((idx & 1) * 4)) & 0xFu) : src[idx];
       const float2 p = qp[idx / group];
@@ -121,8 +122,8 @@ static int embed_tokens(uint32_t map_act, uint32_t map_src, uint32_t locs_tokens
   // rows stored as float32 only: the fp16 mirror of a KV range would go stale
   if (ma->kv16 && dst_start < ma->kv_start + ma->kv_count && ma->kv_start < (uint64_t)dst_start + total) return ADAMAH_ERR_INVALID;
   if (!in_range(src_row0, (uint64_t)V * E, ms->n_elems)) return ADAMAH_ERR_INVALID;
-  const int fmt = ms->dtype == DTYPE_F32 ? 0 : ms->dtype == DTYPE_Q4 ? 1 : ms->dtype == DTYPE_Q8 ? 2 : -1;
-  if (fmt < 0 || (fmt != 0 && (!ms->qp || ms->group_size == 0))) return ADAMAH_ERR_INVALID;
+  const int fmt = ms->dtype == DTYPE_F32 ? 0 : ms->dtype == DTYPE_Q4 ? 1 : ms->dtype == DTYPE_Q8 ? 2 : ms->dtype == DTYPE_BF16 ? 3 : -1;
+  if (fmt < 0 || ((fmt == 1 || fmt == 2) && (!ms->qp || ms->group_size == 0))) return ADAMAH_ERR_INVALID;
   const uint32_t* tl = res_u32(locs_tokens, m);
   if (!tl) return ADAMAH_ERR_INVALID;
   uint32_t tok0 = 0;
@@ -139,7 +140,7 @@ static int embed_tokens(uint32_t map_act, uint32_t map_src, uint32_t locs_tokens
   const dim3 grid(cdiv(total, 256));
 #define EMBED(F) k_embed_tokens<F><<<grid, 256, 0, g.stream>>>((float*)ma->buf, ma->n_elems, ms->buf, ms->n_elems, src_row0, E, V, \
                                                           total, dst_start, tok0, by_val, scale, tl, ms->qp, ms->group_size, m, mail, ticket)
-  if (fmt == 0) EMBED(0); else if (fmt == 1) EMBED(1); else EMBED(2);
+  if (fmt == 0) EMBED(0); else if (fmt == 1) EMBED(1); else if (fmt == 2) EMBED(2); else EMBED(3);
 #undef EMBED
   count_launch();
   return check_launch();

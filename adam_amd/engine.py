@@ -94,20 +94,12 @@ class DecodeEngine:
         if A is None:
             from . import adamah as A
         self.gpu, self.cfg, self.A = gpu, cfg, A
-        self.tensors = tensors = dict(tensors)
         self._gpu_fused_topk = bool(gpu_fused_topk)
         self._gpu_approx_rerank = bool(gpu_approx_rerank)
         self._gpu_approx_partial_k = max(1, min(self.SAMPLE_TOPK_MAX, int(gpu_approx_partial_k or self.SAMPLE_TOPK_MAX)))
         self._force_mode = sampling_mode
         self._lm_q4_approx_name = None
-        head = tensors.get('output.weight')
-        if self._gpu_approx_rerank and isinstance(head, QTensor) and head.kind == 'q8_0':
-            # a 4-bit copy of the 8-bit LM head for the shortlist pass, made as the reference makes it: the
-            # dequantised matrix through the 4-bit map's own quantiser with min / max qparams (engine.py:578-583,
-            # :1077-1085, :1100-1110)
-            from .quant import requantize_q4
-            self._lm_q4_approx_name = 'output.weight.q4_approx'
-            tensors[self._lm_q4_approx_name] = requantize_q4(head.dequant())
+        self.tensors = self._take_tensors(tensors)
         self.verbose = verbose
         self._kv_cap = int(kv_cap)
         self._kv_fp16 = bool(kv_fp16)
@@ -152,6 +144,19 @@ class DecodeEngine:
                 self._ls_plan_id = plan_id + 1
 
     # ------------------------------------------------------------------ layout
+    def _take_tensors(self, tensors):
+        """The model's tensors as this engine keeps them."""
+        tensors = dict(tensors)
+        head = tensors.get('output.weight')
+        if self._gpu_approx_rerank and isinstance(head, QTensor) and head.kind == 'q8_0':
+            # a 4-bit copy of the 8-bit LM head for the shortlist pass, made as the reference makes it: the
+            # dequantised matrix through the 4-bit map's own quantiser with min / max qparams (engine.py:578-583,
+            # :1077-1085, :1100-1110)
+            from .quant import requantize_q4
+            self._lm_q4_approx_name = 'output.weight.q4_approx'
+            tensors[self._lm_q4_approx_name] = requantize_q4(head.dequant())
+        return tensors
+
     @staticmethod
     def _qkv_sort_key(n):
         for a, b in (('.attn_q.', '.attn_z0.'), ('.attn_k.', '.attn_z1.'), ('.attn_v.', '.attn_z2.')):
@@ -193,6 +198,21 @@ class DecodeEngine:
             raise RuntimeError("upload_dev failed")
         return h
 
+    def _span(self, name, sz, pos):
+        h = self._up(np.arange(pos, pos + sz))
+        self._ws[name] = (h, sz, pos)
+        self.gpu.register_loc_span(h, 0, pos, sz)
+
+    def _sample_slots(self):
+        """(name, elements) of the workspace slots the LM head and the sampling modes use."""
+        return [('logits', self.cfg.n_vocab), ('sample_token', 1), ('sample_rand', 1),
+                ('sample_fused_idx', self._fused_groups * self.SAMPLE_TOPK_MAX),
+                ('sample_fused_val', self._fused_groups * self.SAMPLE_TOPK_MAX),
+                ('sample_topk_idx', self.SAMPLE_TOPK_MAX), ('sample_topk_val', self.SAMPLE_TOPK_MAX),
+                ('sample_topk_prob', self.SAMPLE_TOPK_MAX), ('sample_short_sel', self.SAMPLE_APPROX_SHORTLIST_MAX),
+                ('sample_exact_idx', self.SAMPLE_APPROX_SHORTLIST_MAX),
+                ('sample_exact_val', self.SAMPLE_APPROX_SHORTLIST_MAX)]
+
     def _alloc_workspace(self):
         c, g = self.cfg, self.gpu
         kv_cap = self._kv_cap
@@ -201,11 +221,7 @@ class DecodeEngine:
         self._ws = {}
         self._fused_groups = (c.n_vocab + self._rows_per_group - 1) // self._rows_per_group
 
-        def span(name, sz, pos):
-            h = self._up(np.arange(pos, pos + sz))
-            self._ws[name] = (h, sz, pos)
-            g.register_loc_span(h, 0, pos, sz)
-
+        span = self._span
         pos = 0
         sc_sz = c.n_head * kv_cap
         span('scores', sc_sz, 0)
@@ -229,14 +245,7 @@ class DecodeEngine:
 
         slots = [('hidden', c.n_embd), ('normed', c.n_embd), ('q', q_dim), ('k', k_dim), ('v', k_dim),
                  ('attn_out', c.n_head * c.head_dim_kv), ('o_proj', c.n_embd), ('gate', c.n_ff),
-                 ('up', c.n_ff), ('act', c.n_ff), ('ffn_out', c.n_embd), ('logits', c.n_vocab),
-                 ('sample_token', 1), ('sample_rand', 1),
-                 ('sample_fused_idx', self._fused_groups * self.SAMPLE_TOPK_MAX),
-                 ('sample_fused_val', self._fused_groups * self.SAMPLE_TOPK_MAX),
-                 ('sample_topk_idx', self.SAMPLE_TOPK_MAX), ('sample_topk_val', self.SAMPLE_TOPK_MAX),
-                 ('sample_topk_prob', self.SAMPLE_TOPK_MAX), ('sample_short_sel', self.SAMPLE_APPROX_SHORTLIST_MAX),
-                 ('sample_exact_idx', self.SAMPLE_APPROX_SHORTLIST_MAX),
-                 ('sample_exact_val', self.SAMPLE_APPROX_SHORTLIST_MAX),
+                 ('up', c.n_ff), ('act', c.n_ff), ('ffn_out', c.n_embd), *self._sample_slots(),
                  ('normed2', c.n_embd)]
         for name, sz in slots:
             span(name, sz, pos); pos += sz
@@ -309,6 +318,10 @@ class DecodeEngine:
         g.register_row_base_span(self._ao_rows_h, 0, pos_ao, c.n_head, c.head_dim_kv, c.head_dim_kv)
 
         self._hid_locs = np.arange(self._ws['hidden'][2], self._ws['hidden'][2] + c.n_embd, dtype=np.uint32)
+        self._alloc_sample_handles()
+        self._ws_total = pos
+
+    def _alloc_sample_handles(self):
         self._sample_locs = np.array([self._ws['sample_token'][2]], dtype=np.uint32)
         self._rand_locs = np.array([self._ws['sample_rand'][2]], dtype=np.uint32)
         self._sample_fused_base_h = self._up([self._ws['sample_fused_idx'][2]])
@@ -328,7 +341,6 @@ class DecodeEngine:
         self._sample_fused_partial_n = 0
         self._sample_repeat_ids = np.zeros(self.SAMPLE_REPEAT_MAX, np.uint32)
         self._sample_repeat_ids_h = self._up(self._sample_repeat_ids)
-        self._ws_total = pos
 
     # ------------------------------------------------------------------ chunked prefill: workspace
     def _alloc_chunk_slots(self, pos):
@@ -655,27 +667,11 @@ class DecodeEngine:
         return [int(t) for t in self.gpu.token_wait(ticket, m)]
 
     # ------------------------------------------------------------------ forward
-    def _forward(self, tok, pos, sample=True, sample_cfg=None, sample_prev=(), from_device=False, on_token=None,
-                 sample_mode=None, return_logits=False):
-        """One decode step; op order of reference engine.py:2971-3402 (default discrete-GPU path).
-        `sample_mode`: the LM-head / sampling tail to issue (reference engine.py:3318-3640); None picks
-        'gpu_fused_topk' for a sampling configuration and 'gpu_matvec_argmax' otherwise, as before the other
-        modes existed.  `return_logits`: the full logits (final soft-cap applied) are computed and returned.
-        `from_device`: the input token is the one the previous step's LM head left in the token slot (`tok` is
-        not looked at); its embedding row is gathered on the device.  `on_token` (with `from_device`): called with
-        that token once it has reached the host -- after the layers have been issued, before the LM head's ops are
-        (their repeat-penalty list may depend on it); returning False ends the step there."""
-        c, g, A, ws = self.cfg, self.gpu, self.A, self.WS_MAP
-        q_dim, k_dim = c.n_head * c.head_dim, c.n_head_kv * c.head_dim_kv
-        seq_len = pos + 1
-        W = self._ws
-        hid_h, normed_h, q_h, k_h, v_h = (W[n][0] for n in ('hidden', 'normed', 'q', 'k', 'v'))
-        ao_h, op_h, n2_h, gate_h, up_h, act_h, ffn_h = (
-            W[n][0] for n in ('attn_out', 'o_proj', 'normed2', 'gate', 'up', 'act', 'ffn_out'))
-        alias_fast = self._sched != 'legacy'
-
+    def _stage_token(self, tok, from_device):
+        """What a step needs from the host for its input token, ahead of the batch."""
+        c, g = self.cfg, self.gpu
         if from_device:
-            feed = self._token_feed()
+            self._token_feed()
         elif self._tied:
             np.add(self._emb_base, np.uint32(tok * c.n_embd), out=self._emb_locs)
             g.upload_dev(self._emb_locs, handle=self._emb_gather_h)
@@ -683,10 +679,13 @@ class DecodeEngine:
             row = self.tensors['token_embd.weight'].row(tok)
             if c.emb_scale != 1.0:
                 row = row * np.float32(c.emb_scale)
-            g.scatter(ws, self._hid_locs, row)
+            g.scatter(self.WS_MAP, self._hid_locs, row)
 
-        g.batch_begin()
+    def _issue_embedding(self, from_device):
+        c, g, A, ws, W = self.cfg, self.gpu, self.A, self.WS_MAP, self._ws
+        hid_h = W['hidden'][0]
         if from_device:     # (the same launch hands the token to the host: _wait_tokens(self._feed_ticket))
+            feed = self._feed
             self._feed_ticket = g.embed_post_tokens_dev(ws, feed['src'][0], feed['tok_h'], feed['src'][1],
                                                         int(self._hid_locs[0]), 1, c.n_embd, c.n_vocab, float(c.emb_scale))
         elif self._tied:
@@ -696,6 +695,17 @@ class DecodeEngine:
             g.map_scatter_dev(ws, hid_h, c.n_embd, src_h)
             if c.emb_scale != 1.0:
                 g.map_broadcast_dev(ws, A.OP_MUL, hid_h, W['emb_scale'][0], hid_h, c.n_embd)
+
+    def _issue_layers(self, pos):
+        """The layers of a step at position `pos` and the output norm: the registered plan, or op by op."""
+        c, g, A, ws = self.cfg, self.gpu, self.A, self.WS_MAP
+        q_dim, k_dim = c.n_head * c.head_dim, c.n_head_kv * c.head_dim_kv
+        seq_len = pos + 1
+        W = self._ws
+        hid_h, normed_h, q_h, k_h, v_h = (W[n][0] for n in ('hidden', 'normed', 'q', 'k', 'v'))
+        ao_h, op_h, n2_h, gate_h, up_h, act_h, ffn_h = (
+            W[n][0] for n in ('attn_out', 'o_proj', 'normed2', 'gate', 'up', 'act', 'ffn_out'))
+        alias_fast = self._sched != 'legacy'
 
         for L in range(c.n_layer if self._plan_id is None else 0):
             p = f'blk.{L}'
@@ -752,6 +762,23 @@ class DecodeEngine:
             self._rms(hid_h, 'output_norm.weight', normed_h, 1, c.n_embd)
         else:
             g.decode_step(self._plan_id, pos, seq_len)
+
+    def _forward(self, tok, pos, sample=True, sample_cfg=None, sample_prev=(), from_device=False, on_token=None,
+                 sample_mode=None, return_logits=False):
+        """One decode step; op order of reference engine.py:2971-3402 (default discrete-GPU path).
+        `sample_mode`: the LM-head / sampling tail to issue (reference engine.py:3318-3640); None picks
+        'gpu_fused_topk' for a sampling configuration and 'gpu_matvec_argmax' otherwise, as before the other
+        modes existed.  `return_logits`: the full logits (final soft-cap applied) are computed and returned.
+        `from_device`: the input token is the one the previous step's LM head left in the token slot (`tok` is
+        not looked at); its embedding row is gathered on the device.  `on_token` (with `from_device`): called with
+        that token once it has reached the host -- after the layers have been issued, before the LM head's ops are
+        (their repeat-penalty list may depend on it); returning False ends the step there."""
+        c, g, ws, W = self.cfg, self.gpu, self.WS_MAP, self._ws
+        normed_h = W['normed'][0]
+        self._stage_token(tok, from_device)
+        g.batch_begin()
+        self._issue_embedding(from_device)
+        self._issue_layers(pos)
         if from_device and on_token is not None and not on_token(self._wait_tokens(self._feed_ticket)[0]):
             g.batch_end()
             return
@@ -766,11 +793,7 @@ class DecodeEngine:
         if mode == 'gpu_fused_topk':
             self._sample_fused_topk(sample_cfg, sample_prev, normed_h)
         elif mode == 'gpu_matvec_argmax':
-            fn = (g.map_matvec_argmax_t_xq8_dev if self._kind[self._lm_name] == 'q8'
-                  else g.map_matvec_argmax_t_xq4_dev)
-            fn(ws, self._map_of[self._lm_name], normed_h, self._wh[self._lm_name],
-               W['sample_fused_idx'][0], W['sample_fused_val'][0], W['sample_token'][0],
-               c.n_embd, c.n_vocab, self._rows_per_group)
+            self._issue_argmax(normed_h)
             self._sample_token_ready = True
         elif mode == 'gpu_approx_rerank':
             self._issue_approx_shortlist(sample_cfg, sample_prev, normed_h)
@@ -783,6 +806,15 @@ class DecodeEngine:
             return g.gather(ws, self._logit_locs).view(np.float32).copy()
         return None
 
+    def _issue_argmax(self, normed_h):
+        c, g, W = self.cfg, self.gpu, self._ws
+        fn = g.map_matvec_argmax_t_xq8_dev if self._kind[self._lm_name] == 'q8' else g.map_matvec_argmax_t_xq4_dev
+        fn(self.WS_MAP, self._map_of[self._lm_name], normed_h, self._wh[self._lm_name], W['sample_fused_idx'][0],
+           W['sample_fused_val'][0], W['sample_token'][0], c.n_embd, c.n_vocab, self._rows_per_group)
+
+    def _issue_logits(self, normed_h):
+        self._proj(normed_h, self._lm_name, self._ws['logits'][0], self.cfg.n_embd, self.cfg.n_vocab)
+
     # ------------------------------------------------------------------ LM-head / sampling modes
     def _effective_top_k(self, cfg):
         """Deterministic decoding collapses to top-1 (reference engine.py:1843-1850)."""
@@ -791,13 +823,17 @@ class DecodeEngine:
         k = int(cfg.top_k)
         return 0 if k <= 0 else min(k, self.SAMPLE_TOPK_MAX, self.cfg.n_vocab)
 
+    def _head_argmax_built(self):
+        n = f'map_matvec_argmax_t_x{self._kind[self._lm_name]}_dev'
+        return bool(getattr(self.gpu, '_has_' + n, False)) or hasattr(self.gpu, n)
+
     def _select_sampling_mode(self, cfg):
         """The reference's order of preference (engine.py:3783-3805, predicates :1852-1958) without its host-side
         top-1 mode, which exists for one device family only."""
         g, k = self.gpu, self._effective_top_k(cfg)
         kind = self._kind[self._lm_name]
         has = lambda n: bool(getattr(g, n, False)) or hasattr(g, n.replace('_has_', '', 1))
-        matvec_argmax = (k == 1 and cfg.repeat_penalty == 1.0 and has(f'_has_map_matvec_argmax_t_x{kind}_dev'))
+        matvec_argmax = k == 1 and cfg.repeat_penalty == 1.0 and self._head_argmax_built()
         can_topk = 0 < k <= self.SAMPLE_TOPK_MAX
         fused = self._gpu_fused_topk and can_topk and has(f'_has_map_matvec_topk_t_x{kind}_dev')
         rerank = (k > 1 and self._gpu_approx_rerank and self._lm_q4_approx_name is not None and kind == 'q8'
@@ -856,7 +892,7 @@ class DecodeEngine:
         repeat penalty, top-k, top-p and the draw ('gpu_topk'); reference engine.py:3509-3548."""
         c, g, ws, W = self.cfg, self.gpu, self.WS_MAP, self._ws
         lo_h = W['logits'][0]
-        self._proj(normed_h, self._lm_name, lo_h, c.n_embd, c.n_vocab)
+        self._issue_logits(normed_h)
         self._softcap(lo_h, c.n_vocab)
         if mode == 'gpu_argmax':
             g.map_argmax_dev(ws, lo_h, W['sample_token'][0], c.n_vocab)
@@ -1280,6 +1316,10 @@ class DecodeEngine:
         self.gpu.scatter(self.WS_MAP, np.arange(sc_sz, dtype=np.uint32), np.full(sc_sz, -1e30, np.float32))
         self._sample_token_ready = False
 
+    def _usable_prefix(self, n, n_prompt):
+        """How many of the first n prompt tokens need no prefill because the caches still hold them."""
+        return n if n < n_prompt else 0
+
     # ------------------------------------------------------------------ generate
     def generate(self, token_ids, config=None, forced=None, reuse_prefix=0):
         """Generation with the LM-head / sampling mode the configuration selects (`_select_sampling_mode`: greedy
@@ -1302,9 +1342,7 @@ class DecodeEngine:
                 f"KV cache too small: need {len(token_ids) + config.max_tokens} tokens but "
                 f"kv_cap={self._kv_cap}. Reinitialize with kv_cap>={len(token_ids) + config.max_tokens}.")
         mode = self._select_sampling_mode(config)
-        reuse = max(0, int(reuse_prefix or 0))
-        if reuse >= len(token_ids):
-            reuse = 0
+        reuse = self._usable_prefix(max(0, int(reuse_prefix or 0)), len(token_ids))
         self.reset()
         # (the device-side embedding table of an untied model is filled on first use: before the clock starts)
         ahead = (forced is None and self._lookahead and config.max_tokens > 0

@@ -1,0 +1,250 @@
+"""Sequence mixers of the layered models: what tensors each has, what a sequence keeps of it, and the ops it issues.
+
+A mixer names its input projections (they all read the layer's normed hidden row, so they are stacked into one
+matrix), issues its core op over the rows those projections leave in the `x` rows, and its output projection.  The
+engine (`mixer_engine.MixerEngine`) owns rows, weights, state and cache; a mixer only describes.  Sizes and constants
+come from the model's configuration; the ranks of low-rank projections come from the tensors.
+
+Another mixer is another class with these members:
+  tensors(E)            name -> shape, None where the tensor decides
+  inputs()              names of the stacked input projections, in order
+  vectors()             names of the tensors kept as float32 in the workspace
+  widths(shape)         row buffer -> width it needs
+  state_size(), cache_size()   elements per sequence in the float32 state map / in the key-value cache map
+  const_size()          float32 constants from the configuration (`e.const`)
+  core(e, p, x)         issue the sequence op: x maps an input's name to its column in the `x` rows
+  output(e, p, x, out, epi)    issue the output projection into the rows `out`
+"""
+from dataclasses import dataclass
+
+import numpy as np
+
+
+@dataclass
+class ChannelDelta:
+    """Gated delta rule: short convolutions on q, k, v, unit q and k, one decay per head and key channel (low-rank),
+    per-head norm and a low-rank sigmoid gate on the way out."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+    @classmethod
+    def from_config(cls, d):
+        return cls(*(int(d[n]) for n in ("heads", "kv_heads", "dim", "vdim", "conv")))
+
+    def tensors(self, E):
+        H, KH, D, V, T = self.heads, self.kv_heads, self.dim, self.vdim, self.conv
+        return {"q": (KH * D, E), "k": (KH * D, E), "v": (H * V, E), "b": (H, E), "a1": (None, E), "a2": (H * D, None),
+                "g1": (None, E), "g2": (H * V, None), "o": (E, H * V), "q.conv": (KH * D, T), "k.conv": (KH * D, T),
+                "v.conv": (H * V, T), "A_log": (H,), "dt_bias": (H * D,), "norm": (V,)}
+
+    def inputs(self):
+        return ["q", "k", "v", "b", "a1", "g1"]
+
+    def vectors(self):
+        return ["q.conv", "k.conv", "v.conv", "A_log", "dt_bias", "norm"]
+
+    def widths(self, shape):
+        return {"a": self.heads * self.dim, "g": self.heads * self.vdim, "o": self.heads * self.vdim}
+
+    def _channels(self):
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+    def state_size(self):
+        return self.heads * self.dim * self.vdim + self.conv * self._channels()
+
+    def cache_size(self):
+        return 0
+
+    def const_size(self):
+        return 0
+
+    def core(self, e, p, x):
+        A = e.A
+        decay = e.linear_spec([p + "a2"], src=e.at("x", x["a1"]), out=e.at("a"))
+        gate = e.linear_spec([p + "g2"], src=e.at("x", x["g1"]), out=e.at("g"))
+        s_off = e.take_state(self.state_size())
+        xo, xs = e.at("x", x["q"])
+        oo, os_ = e.at("o")
+        spec = A.DeltaSpec(heads=self.heads, kv_heads=self.kv_heads, dim=self.dim, vdim=self.vdim, taps=self.conv, x=xo,
+                           x_stride=xs, x_b=x["b"] - x["q"], cq=e.vec(p + "q.conv"), ck=e.vec(p + "k.conv"),
+                           cv=e.vec(p + "v.conv"), a_log=e.vec(p + "A_log"), dt_bias=e.vec(p + "dt_bias"), out=oo,
+                           out_stride=os_, state_map=e.STATE_MAP, s_off=s_off,
+                           conv_off=s_off + self.heads * self.dim * self.vdim, seq_stride=e.state_per_seq)
+        e.delta_rule(spec, decay, gate)
+
+    def output(self, e, p, x, out, epi):
+        go, gs = e.at("g")
+        e.linear([p + "o"], src=e.at("o"), out=out, epi=epi,
+                 norm=e.norm(self.heads, e.vec(p + "norm"), self.vdim, gate=(go, gs, e.A.GATE_SIGMOID)))
+
+
+@dataclass
+class ChunkAttention:
+    """Softmax attention over the keys of the query's own chunk, with r1 ln(1 + r2 distance) taken off the scores and
+    values divided by their root mean square; grouped key / value heads, no rotation."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    chunk: int
+    rows: str = "o"
+
+    @classmethod
+    def from_config(cls, d, rows="o"):
+        return cls(int(d["heads"]), int(d["kv_heads"]), int(d["dim"]), int(d["vdim"]), float(d["scale"]),
+                   int(d["mask"]["size"]), rows)
+
+    def tensors(self, E):
+        H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
+        return {"q": (H * D, E), "k": (G * D, E), "v": (G * V, E), "o": (E, H * V), "r1": (H,), "r2": (H,)}
+
+    def inputs(self):
+        return ["q", "k", "v"]
+
+    def vectors(self):
+        return ["r1", "r2"]
+
+    def widths(self, shape):
+        return {self.rows: self.heads * self.vdim}
+
+    def state_size(self):
+        return 0
+
+    def cache_size(self):
+        r8 = lambda n: (n + 7) // 8 * 8
+        return self.kv_heads * self.chunk * (r8(self.dim) + r8(self.vdim))
+
+    def const_size(self):
+        return 0
+
+    def core(self, e, p, x):
+        r8 = lambda n: (n + 7) // 8 * 8
+        off = e.take_cache(self.cache_size())
+        xo, xs = e.at("x")
+        oo, os_ = e.at(self.rows)
+        e.chunk_attention(e.A.ChunkAttnSpec(
+            heads=self.heads, kv_heads=self.kv_heads, dim=self.dim, vdim=self.vdim, chunk=self.chunk, x=xo, x_stride=xs,
+            x_q=x["q"], x_k=x["k"], x_v=x["v"], r1=e.vec(p + "r1"), r2=e.vec(p + "r2"), scale=self.scale, eps=e.cfg.norm_eps,
+            out=oo, out_stride=os_, cache_map=e.CACHE_MAP, k_off=off, v_off=off + self.kv_heads * self.chunk * r8(self.dim),
+            seq_stride=e.cache_per_seq))
+
+    def output(self, e, p, x, out, epi):
+        e.linear([p + "o"], src=e.at(self.rows), out=out, epi=epi)
+
+
+@dataclass
+class Retention:
+    """Linear attention with one fixed decay per head; rotary q and k, per-head norm without weight, silu gate."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: tuple
+    rot_base: float
+    rot_dims: int
+    rows: str = "o"
+
+    @classmethod
+    def from_config(cls, d, rows="o"):
+        c = cls(int(d["heads"]), int(d["dim"]), int(d["vdim"]), tuple(float(v) for v in d["decay"]), float(d["rot"]["base"]),
+                int(d["rot"]["dims"]), rows)
+        if len(c.decay) != c.heads:
+            raise ValueError(f"retention: {len(c.decay)} decays for {c.heads} heads")
+        return c
+
+    def tensors(self, E):
+        H, D, V = self.heads, self.dim, self.vdim
+        return {"q": (H * D, E), "k": (H * D, E), "v": (H * V, E), "g": (H * V, E), "o": (E, H * V)}
+
+    def inputs(self):
+        return ["q", "k", "v", "g"]
+
+    def vectors(self):
+        return []
+
+    def widths(self, shape):
+        return {self.rows: self.heads * self.vdim}
+
+    def state_size(self):
+        return self.heads * self.dim * self.vdim
+
+    def cache_size(self):
+        return 0
+
+    def const_size(self):
+        return self.rot_dims // 2 + self.heads
+
+    def core(self, e, p, x):
+        half = self.rot_dims // 2
+        freq = e.const(np.float64(self.rot_base) ** (-2.0 * np.arange(half) / max(self.rot_dims, 1)))
+        xo, xs = e.at("x")
+        oo, os_ = e.at(self.rows)
+        e.retention(e.A.RetentionSpec(
+            heads=self.heads, dim=self.dim, vdim=self.vdim, rot_dims=self.rot_dims, freq=freq, decay=e.const(self.decay),
+            x=xo, x_stride=xs, x_q=x["q"], x_k=x["k"], x_v=x["v"], out=oo, out_stride=os_, state_map=e.STATE_MAP,
+            s_off=e.take_state(self.state_size()), seq_stride=e.state_per_seq))
+
+    def output(self, e, p, x, out, epi):
+        xo, xs = e.at("x", x["g"])
+        e.linear([p + "o"], src=e.at(self.rows), out=out, epi=epi, norm=e.norm(self.heads, gate=(xo, xs, e.A.GATE_SILU)))
+
+
+@dataclass
+class Parallel:
+    """Two mixers that read the same row; half the sum of their outputs, each normed over the model width."""
+    left: object
+    right: object
+
+    @classmethod
+    def from_config(cls, d):
+        return cls(ChunkAttention.from_config(d["left"], "o"), Retention.from_config(d["right"], "o2"))
+
+    def _both(self):
+        return (("left.", self.left), ("right.", self.right))
+
+    def tensors(self, E):
+        t = {n + "out": (E,) for n, _ in self._both()}
+        for n, m in self._both():
+            t.update({n + k: v for k, v in m.tensors(E).items()})
+        return t
+
+    def inputs(self):
+        return [n + k for n, m in self._both() for k in m.inputs()]
+
+    def vectors(self):
+        return [n + k for n, m in self._both() for k in m.vectors() + ["out"]]
+
+    def widths(self, shape):
+        w = {"y": None, "y2": None}                   # None: the model width
+        for _, m in self._both():
+            w.update(m.widths(shape))
+        return w
+
+    def state_size(self):
+        return self.left.state_size() + self.right.state_size()
+
+    def cache_size(self):
+        return self.left.cache_size() + self.right.cache_size()
+
+    def const_size(self):
+        return self.left.const_size() + self.right.const_size()
+
+    @staticmethod
+    def _cols(x, n):
+        return {k[len(n):]: v for k, v in x.items() if k.startswith(n)}
+
+    def core(self, e, p, x):
+        for n, m in self._both():
+            m.core(e, p + n, self._cols(x, n))
+
+    def output(self, e, p, x, out, epi):
+        assert epi == e.A.EPI_ADD
+        for (n, m), rows in zip(self._both(), ("y", "y2")):
+            m.output(e, p + n, self._cols(x, n), e.at(rows), e.A.EPI_STORE)
+        e.merge("y", "y2", e.vec(p + "left.out"), e.vec(p + "right.out"), out, 0.5)
+
+
+MIXERS = {"channel_delta": ChannelDelta, "parallel": Parallel}

@@ -262,7 +262,7 @@ int adamah_matvec_topk_t_xq4_noalloc_dev(uint32_t map_act, uint32_t map_wt, uint
  * gather of host-made locations for tied ones, engine.py:2993-3010) and only then issues the next step.
  * embed_tokens: for r = 0 .. m-1, with tok_r = the float32 token id at element locs_tokens[r] of map_act, elements
  * [dst_start + r*E, dst_start + (r+1)*E) of map_act = scale * row tok_r of the [V, E] table that starts at element
- * src_row0 of map_src (float32, Q4 or Q8 map; quantised values decoded as map_gather_dev decodes them).  The result
+ * src_row0 of map_src (float32, bfloat16, Q4 or Q8 map; quantised values decoded as map_gather_dev decodes them).  The result
  * is what map_gather_dev + map_scatter_dev + a multiplication by scale give for the same token.  A token id outside
  * [0, V) gives a row of zeros.  The destination must lie outside an fp16 KV range. */
 int adamah_hip_embed_tokens_dev(uint32_t map_act, uint32_t map_src, uint32_t locs_tokens, uint32_t src_row0,
@@ -281,6 +281,69 @@ int adamah_hip_token_post(uint32_t map_id, uint32_t locs_handle, uint32_t n, uin
 int adamah_hip_embed_post_tokens_dev(uint32_t map_act, uint32_t map_src, uint32_t locs_tokens, uint32_t src_row0,
                                      uint32_t dst_start, uint32_t m, uint32_t E, uint32_t V, float scale, uint32_t* ticket);
 int adamah_hip_token_wait(uint32_t ticket, float* out, uint32_t n);
+/* ---- layered mixers over bfloat16 weights: no counterpart in the reference ----------------------------------------
+ * A spec handle is an uploaded struct of 32-bit words (map_upload_dev of sizeof(struct) bytes); the library reads its
+ * host copy, checks every range before it launches, and passes the struct to the kernels by value.  Offsets are
+ * element offsets: into the float32 activation map unless said otherwise.  "Rows" are tokens; their buffers are
+ * row-major with the stride the spec names. */
+
+/* y = W . f(x) for `rows` rows, W [n, k] in a bfloat16 map, its rows k_stride apart (a multiple of 64, zeros beyond k).
+ * f: groups = 0: nothing.  Else the row is cut into `groups` equal runs, each divided by sqrt(mean of squares + eps),
+ * then multiplied by the weight (wt_len = 0: none; wt_len < k: repeated) and by the gate (gate_act 1: sigmoid, 2: silu,
+ * of the element at gate + row * gate_stride).  Rows > 1 go through the operand map (bfloat16: bfloat16 matrix
+ * instructions, float32: float32 ones) at `opnd`, rows k_stride apart; ready = 1: they are there already.
+ * epi 0: out = y.  1: out += y.  2: W holds 16 gate rows, their 16 up rows, and so on; silu(gate) * up goes to `out`
+ * (one row) or to the operand map at out_opnd (more rows), n / 2 columns. */
+typedef struct AdamahLinearSpec {
+  uint32_t w, n, k, k_stride, src, src_stride, groups;
+  float eps;
+  uint32_t wt, wt_len, gate, gate_stride, gate_act, opnd, ready, out, out_stride, epi, out_opnd, out_opnd_stride;
+} AdamahLinearSpec;
+/* h_rows: 0, or a handle that names the source row of each row. */
+int adamah_linear_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, uint32_t h_spec, uint32_t h_rows, uint32_t rows);
+/* The same (epi 0), then float(arg-max of row r) to element dst[r] of the activation map (h_dst: `rows` offsets). */
+int adamah_linear_argmax_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, uint32_t h_spec, uint32_t h_dst, uint32_t rows);
+
+/* dst += scale * (a / rms(a) * wa + b / rms(b) * wb) per row. */
+typedef struct AdamahMergeSpec { uint32_t a, b, stride, wa, wb, dst, dst_stride, dim; float eps, scale; } AdamahMergeSpec;
+int adamah_merge_norm_dev(uint32_t map_act, uint32_t h_spec, uint32_t rows);
+
+/* The three sequence mixers below take `rows` consecutive tokens of one sequence (n_seq = 1, slot seq0) at positions
+ * pos .. pos + rows - 1, or one token of each of n_seq sequences (slots seq0 .. seq0 + n_seq - 1), all at position pos.
+ * x: the rows' projections, [rows, x_stride].  State lives in a map of its own, slot s at s * seq_stride; a sequence
+ * that starts (pos = 0) does not read it, so a slot can be handed to another sequence as it is. */
+
+/* Gated delta rule with a decay per head and key channel.  x row: q, k [kv_heads, dim], v [heads, vdim] (before the
+ * convolution of `taps` taps and silu), then at x_b the heads' step sizes before the sigmoid.  The decay's and the
+ * output gate's low-rank second factors are linear ops (h_decay -> a rows [heads * dim], h_gate -> gate rows
+ * [heads * vdim], epi 0) whose sources lie in the x rows.  Conv weights: [channels, taps] at cq, ck, cv. */
+typedef struct AdamahDeltaSpec {
+  uint32_t heads, kv_heads, dim, vdim, taps, x, x_stride, x_b, cq, ck, cv, a_log, dt_bias, out, out_stride;
+  uint32_t state_map, s_off, conv_off, seq_stride;
+} AdamahDeltaSpec;
+int adamah_delta_rule_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, uint32_t h_spec, uint32_t h_decay, uint32_t h_gate,
+                          uint32_t n_seq, uint32_t rows, uint32_t seq0, uint32_t pos);
+
+/* Retention: S = decay_h S + k v^T, o = S^T q.  x row: q, k [heads, dim], v [heads, vdim].  The first rot_dims
+ * dimensions of q and k are rotated by position * freq[i], dimension i paired with i + rot_dims / 2 (freq: rot_dims / 2
+ * values); k is scaled by dim^-1/2. */
+typedef struct AdamahRetentionSpec {
+  uint32_t heads, dim, vdim, rot_dims, freq, decay, x, x_stride, x_q, x_k, x_v, out, out_stride;
+  uint32_t state_map, s_off, seq_stride;
+} AdamahRetentionSpec;
+int adamah_retention_dev(uint32_t map_act, uint32_t h_spec, uint32_t n_seq, uint32_t rows, uint32_t seq0, uint32_t pos);
+
+/* Softmax attention over the keys of the query's own chunk (floor(i / chunk), counted from the sequence's start):
+ * score = (q . k) * scale - r1_h * ln(1 + r2_h * distance); values are divided by their root mean square first and
+ * cached so.  The cache map (float32 or bfloat16) holds a chunk per slot: keys [kv_heads, chunk, d8] at k_off, values
+ * [kv_heads, chunk, v8] at v_off, d8 / v8 = dim / vdim rounded up to 8, token at place position % chunk. */
+typedef struct AdamahChunkAttnSpec {
+  uint32_t heads, kv_heads, dim, vdim, chunk, x, x_stride, x_q, x_k, x_v, r1, r2;
+  float scale, eps;
+  uint32_t out, out_stride, cache_map, k_off, v_off, seq_stride;
+} AdamahChunkAttnSpec;
+int adamah_chunk_attention_dev(uint32_t map_act, uint32_t h_spec, uint32_t n_seq, uint32_t rows, uint32_t seq0, uint32_t pos);
+
 /* ---- measurement and test helpers: not part of the op surface ------------------------------------
  * Nothing a model engine calls.  bench.py times launches with the stopwatch and calibrates profiler counters
  * with the probe; the parity tests read back what the kernels see through the other two. */

@@ -25,6 +25,8 @@ quantiser's ``round()`` tie direction (implementation-defined in GLSL).
 """
 import numpy as np
 
+from .mixer_ops_np import MixerOps
+
 ERR_BACKEND, ERR_MEMORY, ERR_INVALID, ERR_NOT_FOUND = -1, -2, -3, -4
 DTYPE_F32, DTYPE_BF16, DTYPE_Q8, DTYPE_Q4, DTYPE_Q6 = 0, 1, 2, 3, 4
 MAX_MAPS = 16
@@ -43,12 +45,14 @@ class _Map:
         self.group_size = group_size if dtype in (DTYPE_Q8, DTYPE_Q4, DTYPE_Q6) else 0
         if dtype == DTYPE_F32:
             self.data = np.zeros(self.n, np.float32)
+        elif dtype == DTYPE_BF16:
+            self.data = np.zeros(self.n, np.uint16)                      # bit patterns
         elif dtype == DTYPE_Q8:
             self.data = np.zeros(((self.n + 3) // 4) * 4, np.uint8)      # one code per byte
         elif dtype == DTYPE_Q4:
             self.data = np.zeros(((self.n + 7) // 8) * 4, np.uint8)      # two codes per byte
         else:
-            raise NotImplementedError("oracle covers F32, Q8 and Q4 maps only")
+            raise NotImplementedError("oracle covers F32, BF16, Q8 and Q4 maps only")
         self.n_groups = 0
         self.scale = self.zp = None
         if self.group_size > 0:
@@ -99,7 +103,7 @@ class _Map:
         return w
 
 
-class NumpyAdamah:
+class NumpyAdamah(MixerOps):
     """CPU oracle with the reference binding's method surface."""
 
     DTYPE_F32, DTYPE_BF16, DTYPE_Q8, DTYPE_Q4, DTYPE_Q6 = 0, 1, 2, 3, 4
@@ -219,6 +223,8 @@ class NumpyAdamah:
             self._quantise_q4(m, idx, np.ascontiguousarray(data, np.float32).reshape(-1)[:idx.size])
         elif m.dtype == DTYPE_Q8:
             m.data[idx] = np.ascontiguousarray(data).view(np.uint8).reshape(-1)[:idx.size]
+        elif m.dtype == DTYPE_BF16:
+            m.data[idx] = np.ascontiguousarray(data).view(np.uint16).reshape(-1)[:idx.size]
         else:
             m.data[idx] = self._kv_round(map_id, idx, np.ascontiguousarray(data).view(np.float32).reshape(-1)[:idx.size])
         m.cache.clear()
