@@ -157,7 +157,7 @@ class MixerEngine(DecodeEngine):
                 width[n] = max(width.get(n, 0), E if v is None else v)
         self._rows = {}
         for n, w in width.items():
-            w = _up_to(w, 4)
+            w = w if n == "hidden" else _up_to(w, 4)      # (the embedding op writes its rows back to back)
             self._rows[n] = (take(M * w), w)
         self._rows["act"] = (take(_up_to(max(ff, default=0), 16)), _up_to(max(ff, default=0), 16))
         self._rows["logit_rows"] = (take(max(self.LOGIT_ROWS, self._batch) * c.n_vocab), c.n_vocab)
@@ -562,7 +562,7 @@ class MixerEngine(DecodeEngine):
                 width[n] = max(width.get(n, 0), E if v is None else v)
         self._rows = {}
         for n, w in width.items():
-            w = _up_to(w, 4)
+            w = w if n == "hidden" else _up_to(w, 4)      # (the embedding op writes its rows back to back)
             self._rows[n] = (take(M * w), w)
         self._rows["act"] = (take(_up_to(max(ff, default=0), 16)), _up_to(max(ff, default=0), 16))
         self._rows["logit_rows"] = (take(max(self.LOGIT_ROWS, self._batch) * c.n_vocab), c.n_vocab)

@@ -125,3 +125,41 @@ def make_model(cfg, seed=0, sigma=0.02, workers=None):
         for (name, _, _), qt in zip(jobs, ex.map(lambda j: _gen(j[0], j[1], seed, sigma, j[2]), jobs)):
             t[name] = qt
     return t
+
+
+def mixer_config(width, ff, heads, head_dim, kv_heads, n_layer=4, n_vocab=32768, chunk=8192):
+    """A layered mixer model with the proportions of a real one: three delta-rule layers to one parallel layer (chunk
+    attention with grouped heads beside retention), head sizes of 128."""
+    from .mixers import ChannelDelta, ChunkAttention, Parallel, Retention
+    from .models import MixerConfig, MixerLayer
+    layers = []
+    for i in range(n_layer):
+        if i % 4 != 2:
+            m = ChannelDelta(heads, heads, head_dim, head_dim, 4)
+        else:
+            decay = tuple(1.0 - 2.0 ** -(5 + 7 * h / max(heads - 1, 1)) for h in range(heads))
+            m = Parallel(ChunkAttention(heads, kv_heads, head_dim, head_dim, head_dim ** -0.5, chunk, "o"),
+                         Retention(heads, head_dim, head_dim, decay, 1e4, head_dim, "o2"))
+        layers.append(MixerLayer(m, ff))
+    return MixerConfig(arch="Vomotar", n_vocab=n_vocab, n_embd=width, norm_groups=4, norm_eps=1e-6, layers=layers)
+
+
+def make_mixer_model(cfg, seed=0, rank=None):
+    """dict name -> uint16 bfloat16 patterns, random.  Matrices are cut from one pool of normal numbers (what they hold
+    does not change what a step costs)."""
+    from .safetensors_file import f32_to_bf16
+    rng = np.random.default_rng(seed)
+    pool = rng.standard_normal(1 << 24, dtype=np.float32)
+    rank = rank or 128
+    out = {}
+    for n, shape in cfg.tensors().items():
+        shape = tuple(rank if d is None else d for d in shape)
+        size = int(np.prod(shape))
+        at = int(rng.integers(0, pool.size))
+        w = np.resize(np.roll(pool, -at) if size >= pool.size else np.concatenate([pool[at:at + size], pool[:max(0, at + size - pool.size)]]), shape)
+        if len(shape) == 1:
+            w = {"A_log": -2.0 + 0.5 * w, "dt_bias": -3.0 + 0.5 * w, "r1": 0.5 + 0.1 * w, "r2": 0.3 + 0.05 * w}.get(n.split(".")[-1], 1.0 + 0.1 * w)
+        elif not n.endswith(".conv") and n != "embed":
+            w = w * np.float32(shape[-1] ** -0.5)
+        out[n] = f32_to_bf16(np.asarray(w, np.float32))
+    return out

@@ -413,6 +413,77 @@ def measure_lockstep(gpu, A, DecodeEngine, cfg, tensors, batch, n_prompt, steps,
             "ms_per_step": round(st["decode_s"] / steps * 1e3, 3)}
 
 
+MIXER_SIZES = {"2048": dict(width=2048, ff=8192, heads=16, head_dim=128, kv_heads=8),
+               "4096": dict(width=4096, ff=14336, heads=32, head_dim=128, kv_heads=8)}
+
+
+def measure_mixers(gpu, A, synth, DecodeEngine, steps, warmup, n_prompt, sizes, chunk=None, only=None):
+    """Layered mixer model (Vomotar design, bfloat16 weights) beside the Llama shape (Q4_0 body, Q8_0 head) of equal
+    width, feed-forward, heads, depth and vocabulary: prefill of an n_prompt-token random prompt and bs = 1 greedy decoding
+    behind it, both with one step of lookahead.  Four layers; a step's bytes are the weights read once, the states
+    read and written and the visible keys and values; a prompt's work is two operations per weight and token."""
+    from adam_amd.engine import ModelConfig
+    from adam_amd.mixer_engine import MixerEngine
+    out = {}
+    for name in sizes:
+        sz = MIXER_SIZES[name]
+        row = {}
+        if only in (None, "mixer"):
+            cfg = synth.mixer_config(**sz)
+            W = synth.make_mixer_model(cfg)
+            eng = MixerEngine(gpu, cfg, W, A=A, prefill_chunk=chunk or 2048)
+            prompt = [int(t) for t in np.random.default_rng(0).integers(0, cfg.n_vocab, n_prompt)]
+            eng.prefill(prompt)                                         # warm-up: allocations, code objects
+            eng.reset()
+            gpu.sync()
+            t0 = time.perf_counter()
+            eng.prefill(prompt)
+            gpu.sync()
+            pre = time.perf_counter() - t0
+            pos, runs = n_prompt, []
+
+            def run(n):
+                nonlocal pos
+                for _ in range(n):
+                    eng._forward(None, pos, from_device=True)
+                    eng._wait_tokens(eng._feed_ticket)
+                    pos += 1
+            run(warmup)
+            for _ in range(3):
+                gpu.sync()
+                gpu.reset_native_stats()
+                t0 = time.perf_counter()
+                run(steps)
+                gpu.sync()
+                runs.append(time.perf_counter() - t0)
+            launches = gpu.get_native_stats()["dispatch_count"] / steps
+            params = sum(w.size for n, w in W.items() if w.ndim == 2 and n != "embed" and not n.endswith(".conv"))
+            att = sum(2 * L.mixer.left.kv_heads * (L.mixer.left.dim + L.mixer.left.vdim) * (pos % L.mixer.left.chunk)
+                      for L in cfg.layers if hasattr(L.mixer, "left"))
+            step_bytes = 2 * params + 8 * sum(L.mixer.state_size() for L in cfg.layers) + att
+            dt = sorted(runs)[1] / steps
+            row["mixer"] = {"prefill_tok/s": round(n_prompt / pre, 1), "prefill_TFLOP/s": round(2e-12 * params * n_prompt / pre, 1),
+                            "decode_tok/s": round(1 / dt, 1), "ms_per_step": round(1e3 * dt, 4), "step_MB": round(step_bytes / 1e6, 1),
+                            "frac_of_hbm_peak": round(step_bytes / dt / 1e9 / HBM_PEAK_GBPS, 4), "launches_per_token": round(launches, 1)}
+            log(f"mixer {name}: {row['mixer']}")
+            del eng, W
+        if only in (None, "llama"):
+            cfg = ModelConfig(arch="llama", n_vocab=32768, n_embd=sz["width"], n_head=sz["heads"], n_head_kv=sz["kv_heads"], n_layer=4,
+                              n_ff=sz["ff"], head_dim=128, head_dim_kv=128, norm_eps=1e-5, rope_base_global=5e5, rope_base_local=5e5)
+            t = synth.make_model(cfg, seed=0, sigma=0.02)
+            prompt = [int(v) for v in np.random.default_rng(0).integers(0, cfg.n_vocab, n_prompt)]
+            for _ in range(2):                                          # the second run is the warm one
+                m = measure_decode(gpu, A, DecodeEngine, cfg, t, prompt, steps, warmup, "level_batched", chunk or 512)
+            params = sum(int(np.prod(v.shape)) for n, v in t.items() if hasattr(v, "kind"))
+            row["llama_q4_0"] = {"prefill_tok/s": round(n_prompt / m["prefill_s"], 1),
+                                 "prefill_TFLOP/s": round(2e-12 * params * n_prompt / m["prefill_s"], 1), "decode_tok/s": round(m["tok_s"], 1),
+                                 "ms_per_step": round(m["ms_per_step"], 4), "step_MB": round(m["step_bytes"] / 1e6, 1),
+                                 "frac_of_hbm_peak": round(m["tok_s"] / m["ceiling"], 4), "launches_per_token": round(m["launches_per_token"], 1)}
+            log(f"llama {name}: {row['llama_q4_0']}")
+        out[name] = row
+    return {"workload": f"4 layers, {n_prompt}-token prompt, {steps} decode steps (median of three runs)", "sizes": out}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -428,7 +499,8 @@ def main():
                          "reference does; default 512 for llama3-8b, 0 for gemma3-1b); the timed region is the decode "
                          "loop either way")
     ap.add_argument("--batch", type=int, default=16, help="sequences decoded in lockstep (config 5 leg, --only batch)")
-    ap.add_argument("--only", default=None, choices=["roofline", "gemv", "probe", "attention", "gemm", "prefill", "batch"],
+    ap.add_argument("--only", default=None, choices=["roofline", "gemv", "probe", "attention", "gemm", "prefill", "batch", "mixers", "mixers-mixer",
+                                                         "mixers-llama"],
                     help="roofline: just the 28672x4096 GEMV (one kernel row in a rocprofv3 --stats table); "
                          "gemv: that shape, 4096x4096 and 4096x14336; probe: plain read/copy kernels of known "
                          "size (reference points for rocprofv3 --pmc FETCH_SIZE / WRITE_SIZE); attention: GQA "
@@ -436,7 +508,10 @@ def main():
                          "M = 16 and 512 on the Llama-3-8B shapes; prefill: a 512-token prompt of --workload token "
                          "by token and in one chunk (matrix-core matmuls, causal attention in one launch per "
                          "layer); batch: --batch random prompts of --prompt (default 1024) tokens prefilled in "
-                         "chunks of 512, then --steps lockstep decode steps of --workload")
+                         "chunks of 512, then --steps lockstep decode steps of --workload; mixers: the layered mixer model "
+                         "beside the Llama shape of equal size, at two sizes (mixers-mixer / mixers-llama: one of the "
+                         "two)")
+    ap.add_argument("--mixer-size", default=None, choices=list(MIXER_SIZES), help="--only mixers: one width alone")
     ap.add_argument("--skip-reference", action="store_true",
                     help="--only prefill: time the chunked prompt alone (chunks of --prefill-chunk, default the whole "
                          "prompt), without the token-by-token run it is otherwise compared with")
@@ -455,6 +530,13 @@ def main():
         if args.only == "batch" and args.steps == 256:
             args.steps = 128
         print(json.dumps(measure_model_batched(args, A, synth, DecodeEngine)), flush=True)
+        return
+    if args.only and args.only.startswith("mixers"):
+        gpu = A.init()
+        one = args.only.partition("-")[2] or None
+        print(json.dumps({"mixers": measure_mixers(gpu, A, synth, DecodeEngine, min(args.steps, 64), args.warmup, args.prompt or 4032,
+                                                   [args.mixer_size] if args.mixer_size else list(MIXER_SIZES), args.prefill_chunk, one)}), flush=True)
+        gpu.shutdown()
         return
     if args.only:
         gpu = A.init()
