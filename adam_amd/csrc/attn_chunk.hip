@@ -3,8 +3,9 @@
 // A token at position i sees positions floor(i / C) C .. i, so the cache of a sequence is one chunk per layer, token i at
 // place i % C; what a new chunk overwrites is never seen again.  Values are cached divided by their root mean square.
 //
-// One token: k_chunk_attn_step, a workgroup per query head and span of SPAN keys; its own key and value come from the
-// projections (the first query head of a key head stores them).  More than one span: k_chunk_attn_join.
+// One token: k_chunk_attn_step, a workgroup per key head (or RG of its query heads) and span of keys, every key and value
+// read once for all of them; the token's own key and value come from the projections, and the last span's workgroup
+// stores them.  More than one span: k_chunk_attn_join.
 //
 // A portion of a prompt: k_chunk_attn_stage lays the keys the portion sees -- what the cache holds of the first token's
 // chunk, then the portion's own -- out as matrix operands, K [np, dp] and V transposed [vp, np]; k_chunk_attn_keep then
@@ -18,7 +19,7 @@
 namespace adamah {
 
 typedef AdamahChunkAttnSpec ASpec;
-#define SPAN 512u
+#define MAX_SPANS 64u
 #define ATT_MASKED (-1.0e30f)
 
 __device__ __forceinline__ float wsumf(float v) {
@@ -26,120 +27,190 @@ __device__ __forceinline__ float wsumf(float v) {
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
   return v;
 }
-template <class T> __device__ __forceinline__ void load8(const T* p, float (&o)[8]);
-template <> __device__ __forceinline__ void load8<float>(const float* p, float (&o)[8]) {
-  const float4 a = *(const float4*)p, b = *(const float4*)(p + 4);
-  o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
-}
-template <> __device__ __forceinline__ void load8<bf16_t>(const bf16_t* p, float (&o)[8]) {
-  const uint4 a = *(const uint4*)p;
-  o[0] = bf_lo(a.x); o[1] = bf_hi(a.x); o[2] = bf_lo(a.y); o[3] = bf_hi(a.y);
-  o[4] = bf_lo(a.z); o[5] = bf_hi(a.z); o[6] = bf_lo(a.w); o[7] = bf_hi(a.w);
-}
+// Eight consecutive elements as they are stored, and as numbers.
+template <class T> struct Eight;
+template <> struct Eight<float> {
+  float4 a, b;
+  __device__ __forceinline__ void zero() { a = b = make_float4(0, 0, 0, 0); }
+  __device__ __forceinline__ void load(const float* p) { a = *(const float4*)p; b = *(const float4*)(p + 4); }
+  __device__ __forceinline__ void set(const float (&x)[8]) { a = make_float4(x[0], x[1], x[2], x[3]); b = make_float4(x[4], x[5], x[6], x[7]); }
+  __device__ __forceinline__ void get(float (&o)[8]) const { o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w; }
+};
+template <> struct Eight<bf16_t> {
+  uint4 a;
+  __device__ __forceinline__ void zero() { a = make_uint4(0, 0, 0, 0); }
+  __device__ __forceinline__ void load(const bf16_t* p) { a = *(const uint4*)p; }
+  __device__ __forceinline__ void set(const float (&x)[8]) {
+    union { bf8_t v; uint4 u; } c;
+#pragma unroll
+    for (int i = 0; i < 8; i++) c.v[i] = (bf16_t)x[i];
+    a = c.u;
+  }
+  __device__ __forceinline__ void get(float (&o)[8]) const {
+    o[0] = bf_lo(a.x); o[1] = bf_hi(a.x); o[2] = bf_lo(a.y); o[3] = bf_hi(a.y);
+    o[4] = bf_lo(a.z); o[5] = bf_hi(a.z); o[6] = bf_lo(a.w); o[7] = bf_hi(a.w);
+  }
+};
 
 // ---- one token ------------------------------------------------------------------------------------------------------
-// grid (heads, spans, sequences).  part: per (sequence, head, span) vdim + 2 floats {max, sum, values}, used when
-// spans > 1.
-template <class T>
+// grid (key heads * groups of RG query heads, spans, sequences).  Sixteen lanes share a key: lane l16 holds columns
+// 8 l16 + 128 c; a wave takes 4 KI keys at a time, their keys and values asked for together.  part: per (sequence, head,
+// span) vdim + 2 floats {max, sum, values}, used when there is more than one span.
+template <class T, int NC, int RG, int KI>
 __global__ void __launch_bounds__(256)
-k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq0, uint32_t pos) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];
-  __shared__ float sh[12];
+k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq0, uint32_t pos, uint32_t span, uint32_t parts) {
+  __shared__ float qb[RG][128 * NC];
+  __shared__ float ob[4][RG][128 * NC], ml[4][RG][2];
   const uint32_t D = s.dim, V = s.vdim, D8 = (D + 7u) & ~7u, V8 = (V + 7u) & ~7u, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
-  const uint32_t h = blockIdx.x, row = blockIdx.z, rep = s.heads / s.kv_heads, kv = h / rep;
-  const uint32_t n = pos % s.chunk + 1u, k0 = blockIdx.y * SPAN, k1 = min(n, k0 + SPAN);
-  const bool own = k1 == n;                                     // this span ends with the token itself
-  float *q = lds, *sc = q + D8, *vn = sc + SPAN, *red = vn + V8;  // red: [256 / (V8 / 8)][V8]
+  const uint32_t row = blockIdx.z, rep = s.heads / s.kv_heads, kv = blockIdx.x / parts, h0 = kv * rep + (blockIdx.x - kv * parts) * RG;
+  const uint32_t nh = min((uint32_t)RG, (kv + 1u) * rep - h0);       // query heads of this workgroup
+  const uint32_t n = pos % s.chunk + 1u, k0 = blockIdx.y * span, k1 = min(n, k0 + span), l16 = lane & 15u, kq = lane >> 4;
   const float* x = act + s.x + (uint64_t)row * s.x_stride;
-  T* K = cache + (uint64_t)(seq0 + row) * s.seq_stride + s.k_off + (uint64_t)kv * s.chunk * D8;
-  T* Vc = cache + (uint64_t)(seq0 + row) * s.seq_stride + s.v_off + (uint64_t)kv * s.chunk * V8;
   const float* xk = x + s.x_k + kv * D;
   const float* xv = x + s.x_v + kv * V;
-  float qk = 0.f, vv = 0.f;
-  for (uint32_t d = tid; d < D8; d += 256u) {
-    const float t = d < D ? x[s.x_q + h * D + d] : 0.f;
-    q[d] = t;
-    if (d < D) qk = fmaf(t, xk[d], qk);
+  T* K = cache + (uint64_t)(seq0 + row) * s.seq_stride + s.k_off + (uint64_t)kv * s.chunk * D8;
+  T* Vc = cache + (uint64_t)(seq0 + row) * s.seq_stride + s.v_off + (uint64_t)kv * s.chunk * V8;
+  const bool own = k1 == n;                                     // this span ends with the token itself
+  float iv = 0.f;
+  if (own) {
+    for (uint32_t d = lane; d < V; d += 64u) iv = fmaf(xv[d], xv[d], iv);
+    iv = 1.0f / sqrtf(wsumf(iv) / (float)V + s.eps);
   }
-  for (uint32_t d = tid; d < V; d += 256u) vv = fmaf(xv[d], xv[d], vv);
-  qk = wsumf(qk); vv = wsumf(vv);
-  if (lane == 0) { sh[wave] = qk; sh[4 + wave] = vv; }
+  for (uint32_t i = tid; i < RG * 128u * NC; i += 256u) {
+    const uint32_t r = i / (128u * NC), d = i - r * (128u * NC);
+    qb[r][d] = (r < nh && d < D) ? x[s.x_q + (h0 + r) * D + d] * s.scale : 0.f;
+  }
+  float r1[RG], r2[RG], mx[RG], sum[RG], o[RG][NC][8];
+#pragma unroll
+  for (int r = 0; r < RG; r++) {
+    const uint32_t h = h0 + min((uint32_t)r, nh - 1u);
+    r1[r] = act[s.r1 + h]; r2[r] = act[s.r2 + h];
+    mx[r] = ATT_MASKED; sum[r] = 0.f;
+#pragma unroll
+    for (int c = 0; c < NC; c++)
+#pragma unroll
+      for (int i = 0; i < 8; i++) o[r][c][i] = 0.f;
+  }
   __syncthreads();
-  qk = (sh[0] + sh[1]) + (sh[2] + sh[3]);
-  const float iv = 1.0f / sqrtf(((sh[4] + sh[5]) + (sh[6] + sh[7])) / (float)V + s.eps);
-  const float r1 = act[s.r1 + h], r2 = act[s.r2 + h];
-  for (uint32_t d = tid; d < V8; d += 256u) vn[d] = d < V ? xv[d] * iv : 0.f;
-  if (own && h % rep == 0) {
+  for (uint32_t kb = k0 + wave * 4u * KI; kb < k1; kb += 16u * KI) {
+    Eight<T> kr[KI][NC], vr[KI][NC];
+#pragma unroll
+    for (int j = 0; j < KI; j++) {
+      const uint32_t key = kb + kq + 4u * j;
+#pragma unroll
+      for (int c = 0; c < NC; c++) {
+        const uint32_t d = l16 * 8u + 128u * c;
+        kr[j][c].zero(); vr[j][c].zero();
+        if (key + 1u < n && key < k1) {
+          if (d < D8) kr[j][c].load(K + (uint64_t)key * D8 + d);
+          if (d < V8) vr[j][c].load(Vc + (uint64_t)key * V8 + d);
+        } else if (key + 1u == n) {
+          float a[8], b[8];
+#pragma unroll
+          for (int i = 0; i < 8; i++) { a[i] = d + i < D ? xk[d + i] : 0.f; b[i] = d + i < V ? xv[d + i] * iv : 0.f; }
+          kr[j][c].set(a); vr[j][c].set(b);
+        }
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < RG; r++) {
+      float sc[KI], top = ATT_MASKED;
+#pragma unroll
+      for (int j = 0; j < KI; j++) sc[j] = 0.f;
+#pragma unroll
+      for (int c = 0; c < NC; c++) {
+        float q[8];
+#pragma unroll
+        for (int i = 0; i < 8; i++) q[i] = qb[r][128u * c + l16 * 8u + i];
+#pragma unroll
+        for (int j = 0; j < KI; j++) {
+          float kk[8];
+          kr[j][c].get(kk);
+#pragma unroll
+          for (int i = 0; i < 8; i++) sc[j] = fmaf(kk[i], q[i], sc[j]);
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < KI; j++) {
+        float a = sc[j];
+        a += __shfl_xor(a, 1, 64); a += __shfl_xor(a, 2, 64); a += __shfl_xor(a, 4, 64); a += __shfl_xor(a, 8, 64);
+        const uint32_t key = kb + kq + 4u * j;
+        sc[j] = key < k1 ? a - r1[r] * logf(fmaf(r2[r], (float)(n - 1u - key), 1.0f)) : ATT_MASKED;
+        top = fmaxf(top, sc[j]);
+      }
+      top = fmaxf(top, __shfl_xor(top, 16, 64)); top = fmaxf(top, __shfl_xor(top, 32, 64));
+      const float nm = fmaxf(mx[r], top), al = expf(mx[r] - nm);
+      mx[r] = nm;
+      sum[r] *= al;
+#pragma unroll
+      for (int c = 0; c < NC; c++)
+#pragma unroll
+        for (int i = 0; i < 8; i++) o[r][c][i] *= al;
+#pragma unroll
+      for (int j = 0; j < KI; j++) {
+        const float p = sc[j] > 0.5f * ATT_MASKED ? expf(sc[j] - nm) : 0.f;
+        sum[r] += p;
+#pragma unroll
+        for (int c = 0; c < NC; c++) {
+          float vv[8];
+          vr[j][c].get(vv);
+#pragma unroll
+          for (int i = 0; i < 8; i++) o[r][c][i] = fmaf(p, vv[i], o[r][c][i]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RG; r++) {                                // the four key groups of a wave, then the waves
+    sum[r] += __shfl_xor(sum[r], 16, 64); sum[r] += __shfl_xor(sum[r], 32, 64);
+    if (lane == 0) { ml[wave][r][0] = mx[r]; ml[wave][r][1] = sum[r]; }
+#pragma unroll
+    for (int c = 0; c < NC; c++)
+#pragma unroll
+      for (int i = 0; i < 8; i++) {
+        float a = o[r][c][i];
+        a += __shfl_xor(a, 16, 64); a += __shfl_xor(a, 32, 64);
+        if (kq == 0) ob[wave][r][128u * c + l16 * 8u + i] = a;
+      }
+  }
+  __syncthreads();
+  for (uint32_t i = tid; i < nh * V; i += 256u) {
+    const uint32_t r = i / V, d = i - r * V, h = h0 + r;
+    const float m4 = fmaxf(fmaxf(ml[0][r][0], ml[1][r][0]), fmaxf(ml[2][r][0], ml[3][r][0]));
+    float a = 0.f, t = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; w++) { const float e = expf(ml[w][r][0] - m4); a = fmaf(e, ob[w][r][d], a); t = fmaf(e, ml[w][r][1], t); }
+    if (gridDim.y == 1) act[s.out + (uint64_t)row * s.out_stride + h * V + d] = a / t;
+    else {
+      float* p = part + (((uint64_t)row * s.heads + h) * gridDim.y + blockIdx.y) * (V + 2u);
+      p[2u + d] = a;
+      if (d == 0) { p[0] = m4; p[1] = t; }
+    }
+  }
+  if (own && h0 == kv * rep) {
     for (uint32_t d = tid; d < D8; d += 256u) K[(uint64_t)(n - 1u) * D8 + d] = (T)(d < D ? xk[d] : 0.f);
     for (uint32_t d = tid; d < V8; d += 256u) Vc[(uint64_t)(n - 1u) * V8 + d] = (T)(d < V ? xv[d] * iv : 0.f);
   }
-  // scores: 16 lanes a key
-  const uint32_t l16 = lane & 15u, kq = lane >> 4, last = own ? k1 - 1u : k1;   // cached keys of the span: [k0, last)
-  for (uint32_t j = k0 + wave * 4u; j < last; j += 16u) {
-    const uint32_t key = j + kq;
-    float a = 0.f;
-    if (key < last)
-      for (uint32_t c = l16 * 8u; c < D8; c += 128u) {
-        float kk[8];
-        load8<T>(K + (uint64_t)key * D8 + c, kk);
-#pragma unroll
-        for (int i = 0; i < 8; i++) a = fmaf(kk[i], q[c + i], a);
-      }
-    a += __shfl_xor(a, 1, 64); a += __shfl_xor(a, 2, 64); a += __shfl_xor(a, 4, 64); a += __shfl_xor(a, 8, 64);
-    if (l16 == 0 && key < last) sc[key - k0] = a * s.scale - r1 * log1pf(r2 * (float)(n - 1u - key));
-  }
-  if (own && tid == 0) sc[k1 - 1u - k0] = qk * s.scale;          // distance 0: ln 1 = 0
-  __syncthreads();
-  float mx = ATT_MASKED, sum = 0.f;
-  for (uint32_t j = tid; j < k1 - k0; j += 256u) mx = fmaxf(mx, sc[j]);
-#pragma unroll
-  for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
-  if (lane == 0) sh[wave] = mx;
-  __syncthreads();
-  mx = fmaxf(fmaxf(sh[0], sh[1]), fmaxf(sh[2], sh[3]));
-  for (uint32_t j = tid; j < k1 - k0; j += 256u) { const float e = expf(sc[j] - mx); sc[j] = e; sum += e; }
-  sum = wsumf(sum);
-  if (lane == 0) sh[8 + wave] = sum;
-  __syncthreads();
-  sum = (sh[8] + sh[9]) + (sh[10] + sh[11]);
-  // values: 8 columns a thread, keys dealt out over the thread groups
-  const uint32_t nc = V8 >> 3, ng = 256u / nc, gi = tid / nc, c8 = (tid - gi * nc) * 8u;
-  float o[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-  if (gi < ng) {
-    for (uint32_t key = k0 + gi; key < last; key += ng) {
-      float t[8];
-      load8<T>(Vc + (uint64_t)key * V8 + c8, t);
-      const float p = sc[key - k0];
-#pragma unroll
-      for (int i = 0; i < 8; i++) o[i] = fmaf(p, t[i], o[i]);
-    }
-#pragma unroll
-    for (int i = 0; i < 8; i++) red[gi * V8 + c8 + i] = o[i];
-  }
-  __syncthreads();
-  const float pw = own ? sc[k1 - 1u - k0] : 0.f;
-  for (uint32_t d = tid; d < V; d += 256u) {
-    float a = pw * vn[d];
-    for (uint32_t gg = 0; gg < ng; gg++) a += red[gg * V8 + d];
-    if (gridDim.y == 1) act[s.out + (uint64_t)row * s.out_stride + h * V + d] = a / sum;
-    else part[(((uint64_t)row * s.heads + h) * gridDim.y + blockIdx.y) * (V + 2u) + 2u + d] = a;
-  }
-  if (gridDim.y > 1 && tid == 0) {
-    float* p = part + (((uint64_t)row * s.heads + h) * gridDim.y + blockIdx.y) * (V + 2u);
-    p[0] = mx; p[1] = sum;
-  }
 }
-__global__ void __launch_bounds__(128)
+__global__ void __launch_bounds__(256)
 k_chunk_attn_join(const ASpec s, float* act, const float* __restrict__ part, uint32_t n_part) {
-  const uint32_t h = blockIdx.x, row = blockIdx.y, V = s.vdim;
+  __shared__ float w[MAX_SPANS];
+  const uint32_t h = blockIdx.x, row = blockIdx.y, V = s.vdim, lane = threadIdx.x;
   const float* p = part + ((uint64_t)row * s.heads + h) * n_part * (V + 2u);
-  float mx = ATT_MASKED, sum = 0.f;
-  for (uint32_t i = 0; i < n_part; i++) mx = fmaxf(mx, p[(uint64_t)i * (V + 2u)]);
-  for (uint32_t i = 0; i < n_part; i++) sum += p[(uint64_t)i * (V + 2u) + 1u] * expf(p[(uint64_t)i * (V + 2u)] - mx);
-  for (uint32_t d = threadIdx.x; d < V; d += 128u) {
+  if (lane < 64u) {
+    const float m = lane < n_part ? p[(uint64_t)lane * (V + 2u)] : ATT_MASKED, l = lane < n_part ? p[(uint64_t)lane * (V + 2u) + 1u] : 0.f;
+    float mx = m;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
+    const float e = lane < n_part ? expf(m - mx) : 0.f;
+    w[lane] = e / wsumf(e * l);
+  }
+  __syncthreads();
+  for (uint32_t d = threadIdx.x; d < V; d += 256u) {
     float a = 0.f;
-    for (uint32_t i = 0; i < n_part; i++) a = fmaf(expf(p[(uint64_t)i * (V + 2u)] - mx), p[(uint64_t)i * (V + 2u) + 2u + d], a);
-    act[s.out + (uint64_t)row * s.out_stride + h * V + d] = a / sum;
+#pragma unroll 8
+    for (uint32_t i = 0; i < n_part; i++) a = fmaf(w[i], p[(uint64_t)i * (V + 2u) + 2u + d], a);
+    act[s.out + (uint64_t)row * s.out_stride + h * V + d] = a;
   }
 }
 
@@ -259,91 +330,130 @@ k_chunk_attn_f32(const ASpec s, float* act, const float* __restrict__ K, const f
     }
 }
 
-// bfloat16 form: keys 32 at a time (two tiles of 16); DK: k-steps of 32 dimensions.
-template <int DK, int NV>
-__global__ void __launch_bounds__(256)
+// bfloat16 form: QT tiles of 16 queries a wave, keys 32 at a time (two tiles of 16); DK: k-steps of 32 dimensions.  Scores
+// and the penalty are kept in powers of two.  A step's values and the next step's keys are in flight under the products.
+template <int DK, int NV, int QT>
+__global__ void __launch_bounds__(256, DK * QT <= 8 && NV * QT <= 16 ? 2 : 1)
 k_chunk_attn_bf16(const ASpec s, float* act, const bf16_t* __restrict__ K, const bf16_t* __restrict__ VT, StageDims sd, uint32_t m, uint32_t pos) {
-  const uint32_t lane = threadIdx.x & 63u, c = lane & 15u, kg = lane >> 4, h = blockIdx.x, kv = h / (s.heads / s.kv_heads);
-  const uint32_t q0 = (blockIdx.y * 4u + (threadIdx.x >> 6)) * 16u;
+  // workgroups land on the eight dies in turn: the query heads of a key head share one; late query tiles, which see more
+  // keys, go with early ones
+  const uint32_t nx = gridDim.x, h = (nx & 7u) == 0u ? (blockIdx.x & 7u) * (nx >> 3) + (blockIdx.x >> 3) : blockIdx.x;
+  const uint32_t ny = gridDim.y, by = blockIdx.y < (ny >> 1) ? blockIdx.y : ny - 1u - (blockIdx.y - (ny >> 1));
+  const uint32_t lane = threadIdx.x & 63u, c = lane & 15u, kg = lane >> 4, kv = h / (s.heads / s.kv_heads);
+  const uint32_t q0 = (by * 4u + (threadIdx.x >> 6)) * 16u * QT;
   if (q0 >= m) return;
-  const uint32_t qr = min(q0 + c, m - 1u), base = pos - sd.past;
-  const uint32_t qj = sd.past + qr, lo = (pos + qr) / s.chunk * s.chunk - base;
-  const uint32_t first = ((pos + q0) / s.chunk * s.chunk - base) & ~31u, end = sd.past + min(q0 + 16u, m);
-  const uint32_t lo_all = (pos + min(q0 + 15u, m - 1u)) / s.chunk * s.chunk - base;    // seen by every query from here ..
-  const float* xq = act + s.x + (uint64_t)qr * s.x_stride + s.x_q + h * s.dim;
-  const bf16_t* kb = K + (uint64_t)kv * sd.np * sd.dp;
-  const bf16_t* vb = VT + (uint64_t)kv * sd.vp * sd.np;
+  const uint32_t base = pos - sd.past, qlast = min(q0 + 16u * QT, m) - 1u;
+  const uint32_t first = ((pos + q0) / s.chunk * s.chunk - base) & ~31u, end = sd.past + qlast + 1u;
+  const uint32_t lo_all = (pos + qlast) / s.chunk * s.chunk - base;        // seen by every query from here to past + q0
+  const bf16_t* kb = K + (uint64_t)kv * sd.np * sd.dp + (uint64_t)c * sd.dp + 8u * kg;
+  const bf16_t* vb = VT + (uint64_t)kv * sd.vp * sd.np + (uint64_t)c * sd.np + 4u * kg;
   const float r1 = act[s.r1 + h], r2 = act[s.r2 + h];
-  bf8_t qh[DK], ql[DK];
+  uint32_t qr[QT], qj[QT], lo[QT];
+  bf8_t qh[QT][DK], ql[QT][DK];
 #pragma unroll
-  for (int t = 0; t < DK; t++)
-#pragma unroll
-    for (int i = 0; i < 8; i++) {
-      const uint32_t d = 32u * t + 8u * kg + i;
-      const float x = d < s.dim ? xq[d] * s.scale : 0.f;
-      qh[t][i] = (bf16_t)x;
-      ql[t][i] = (bf16_t)(x - (float)qh[t][i]);
-    }
-  f4_t o[NV];
-#pragma unroll
-  for (int i = 0; i < NV; i++) o[i] = (f4_t){0, 0, 0, 0};
-  float mx = ATT_MASKED, sum = 0.f;
-  for (uint32_t j0 = first; j0 < end; j0 += 32u) {
-    f4_t a[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
+  for (int g = 0; g < QT; g++) {
+    qr[g] = min(q0 + 16u * g + c, m - 1u);
+    qj[g] = sd.past + qr[g];
+    lo[g] = (pos + qr[g]) / s.chunk * s.chunk - base;
+    const float* xq = act + s.x + (uint64_t)qr[g] * s.x_stride + s.x_q + h * s.dim;
 #pragma unroll
     for (int t = 0; t < DK; t++)
 #pragma unroll
-      for (int u = 0; u < 2; u++) {
-        const bf8_t kk = *(const bf8_t*)(kb + (uint64_t)(j0 + 16u * u + c) * sd.dp + 32u * t + 8u * kg);
-        a[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kk, ql[t], a[u], 0, 0, 0);
-        a[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kk, qh[t], a[u], 0, 0, 0);
+      for (int i = 0; i < 8; i++) {
+        const uint32_t d = 32u * t + 8u * kg + i;
+        const float x = d < s.dim ? xq[d] * (s.scale * 1.44269504f) : 0.f;
+        qh[g][t][i] = (bf16_t)x;
+        ql[g][t][i] = (bf16_t)(x - (float)qh[g][t][i]);
       }
-    const bool all = j0 >= lo_all && j0 + 31u <= sd.past + q0;             // .. to here
-    float t = ATT_MASKED;
+  }
+  f4_t o[QT][NV];
+  float mx[QT], sum[QT];
+#pragma unroll
+  for (int g = 0; g < QT; g++) {
+    mx[g] = ATT_MASKED; sum[g] = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; i++) o[g][i] = (f4_t){0, 0, 0, 0};
+  }
+  bf8_t kf[2][DK];
+  auto keys = [&](uint32_t j0) {
 #pragma unroll
     for (int u = 0; u < 2; u++)
 #pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const uint32_t j = j0 + 16u * u + 4u * kg + i;
-        const bool ok = all || (j >= lo && j <= qj);
-        a[u][i] = ok ? a[u][i] - r1 * __logf(fmaf(r2, (float)(qj - j), 1.0f)) : ATT_MASKED;
-        t = fmaxf(t, a[u][i]);
-      }
-    t = fmaxf(t, __shfl_xor(t, 16, 64)); t = fmaxf(t, __shfl_xor(t, 32, 64));
-    const float nm = fmaxf(mx, t), al = __expf(mx - nm);
-    mx = nm;
-    float ps = 0.f;
-    bf8_t ph, pl;
-#pragma unroll
-    for (int u = 0; u < 2; u++)
-#pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const float p = a[u][i] > 0.5f * ATT_MASKED ? __expf(a[u][i] - nm) : 0.f;
-        ps += p;
-        ph[4 * u + i] = (bf16_t)p;
-        pl[4 * u + i] = (bf16_t)(p - (float)ph[4 * u + i]);
-      }
-    ps += __shfl_xor(ps, 16, 64); ps += __shfl_xor(ps, 32, 64);
-    sum = fmaf(sum, al, ps);
+      for (int t = 0; t < DK; t++) kf[u][t] = *(const bf8_t*)(kb + (uint64_t)(j0 + 16u * u) * sd.dp + 32u * t);
+  };
+  keys(first);
+  for (uint32_t j0 = first; j0 < end; j0 += 32u) {
+    bf4_t vf[NV][2];
 #pragma unroll
     for (int v = 0; v < NV; v++) {
-      const bf16_t* src = vb + (uint64_t)(v * 16u + c) * sd.np + j0 + 4u * kg;
-      const bf4_t v0 = *(const bf4_t*)src, v1 = *(const bf4_t*)(src + 16);
-      const bf8_t vv = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-      o[v] *= al;
-      o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pl, o[v], 0, 0, 0);
-      o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, ph, o[v], 0, 0, 0);
+      vf[v][0] = *(const bf4_t*)(vb + (uint64_t)v * 16u * sd.np + j0);
+      vf[v][1] = *(const bf4_t*)(vb + (uint64_t)v * 16u * sd.np + j0 + 16u);
+    }
+    f4_t a[QT][2];
+#pragma unroll
+    for (int g = 0; g < QT; g++)
+#pragma unroll
+      for (int u = 0; u < 2; u++) {
+        a[g][u] = (f4_t){0, 0, 0, 0};
+#pragma unroll
+        for (int t = 0; t < DK; t++) {
+          a[g][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[u][t], ql[g][t], a[g][u], 0, 0, 0);
+          a[g][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[u][t], qh[g][t], a[g][u], 0, 0, 0);
+        }
+      }
+    if (j0 + 32u < end) keys(j0 + 32u);
+    const bool all = j0 >= lo_all && j0 + 31u <= sd.past + q0;
+#pragma unroll
+    for (int g = 0; g < QT; g++) {
+      const float dist = (float)(int32_t)(qj[g] - j0 - 4u * kg);
+      float t = ATT_MASKED;
+#pragma unroll
+      for (int u = 0; u < 2; u++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          const float pen = r1 * __builtin_amdgcn_logf(fmaf(r2, dist - (float)(16 * u + i), 1.0f));
+          const uint32_t j = j0 + 16u * u + 4u * kg + i;
+          a[g][u][i] = all || (j >= lo[g] && j <= qj[g]) ? a[g][u][i] - pen : ATT_MASKED;
+          t = fmaxf(t, a[g][u][i]);
+        }
+      t = fmaxf(t, __shfl_xor(t, 16, 64)); t = fmaxf(t, __shfl_xor(t, 32, 64));
+      const float nm = fmaxf(mx[g], t), al = __builtin_amdgcn_exp2f(mx[g] - nm);
+      mx[g] = nm;
+      float ps = 0.f;
+      bf8_t ph, pl;
+#pragma unroll
+      for (int u = 0; u < 2; u++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          const float p = all || a[g][u][i] > 0.5f * ATT_MASKED ? __builtin_amdgcn_exp2f(a[g][u][i] - nm) : 0.f;
+          ps += p;
+          ph[4 * u + i] = (bf16_t)p;
+          pl[4 * u + i] = (bf16_t)(p - (float)ph[4 * u + i]);
+        }
+      sum[g] = fmaf(sum[g], al, ps);                       // per lane: the four key groups are added up at the end
+#pragma unroll
+      for (int v = 0; v < NV; v++) {
+        const bf8_t vv = {vf[v][0][0], vf[v][0][1], vf[v][0][2], vf[v][0][3], vf[v][1][0], vf[v][1][1], vf[v][1][2], vf[v][1][3]};
+        o[g][v] *= al;
+        o[g][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pl, o[g][v], 0, 0, 0);
+        o[g][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, ph, o[g][v], 0, 0, 0);
+      }
     }
   }
-  if (q0 + c >= m) return;
-  float* out = act + s.out + (uint64_t)qr * s.out_stride + h * s.vdim;
 #pragma unroll
-  for (int v = 0; v < NV; v++)
+  for (int g = 0; g < QT; g++) {
+    sum[g] += __shfl_xor(sum[g], 16, 64); sum[g] += __shfl_xor(sum[g], 32, 64);
+    if (q0 + 16u * g + c >= m) continue;
+    const float inv = 1.0f / sum[g];
+    float* out = act + s.out + (uint64_t)qr[g] * s.out_stride + h * s.vdim;
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-      const uint32_t d = v * 16u + 4u * kg + i;
-      if (d < s.vdim) out[d] = o[v][i] / sum;
-    }
+    for (int v = 0; v < NV; v++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const uint32_t d = v * 16u + 4u * kg + i;
+        if (d < s.vdim) out[d] = o[g][v][i] * inv;
+      }
+  }
 }
 
 static Scratch g_stage, g_parts;
@@ -351,9 +461,12 @@ void attn_chunk_release() { scratch_free(g_stage); scratch_free(g_parts); }
 
 template <int DK>
 static void launch_bf16(const ASpec& s, float* act, const bf16_t* K, const bf16_t* VT, const StageDims& sd, uint32_t m, uint32_t pos) {
-  const dim3 grid(s.heads, cdiv(m, 64));
   switch (sd.vp / 16u) {
-#define CASE(N) case N: k_chunk_attn_bf16<DK, N><<<grid, 256, 0, g.stream>>>(s, act, K, VT, sd, m, pos); break
+#define CASE(N)                                                                                                     \
+  case N: {                                                                                                         \
+    constexpr int QT = DK <= 4 && N <= 8 ? 2 : 1;                                                                   \
+    k_chunk_attn_bf16<DK, N, QT><<<dim3(s.heads, cdiv(m, 64 * QT)), 256, 0, g.stream>>>(s, act, K, VT, sd, m, pos); \
+  } break
     CASE(2); CASE(4); CASE(6); CASE(8); CASE(12); CASE(16);
 #undef CASE
   }
@@ -400,20 +513,30 @@ static int run_portion(const ASpec& s, float* act, T* cache, uint32_t m, uint32_
   return check_launch();
 }
 
-template <class T>
-static int run_step(const ASpec& s, float* act, T* cache, uint32_t n_seq, uint32_t seq0, uint32_t pos) {
-  const uint32_t spans = cdiv(pos % s.chunk + 1u, SPAN), V8 = (s.vdim + 7u) & ~7u, D8 = (s.dim + 7u) & ~7u;
-  if (s.chunk > SPAN)      // at its full size from the first step on: a graph may be recording when the second span begins
-    if (int r = scratch_need(g_parts, (size_t)n_seq * s.heads * cdiv(s.chunk, SPAN) * (s.vdim + 2) * 4)) return r;
-  const size_t lds = ((size_t)D8 + SPAN + V8 + (256 / (V8 / 8)) * V8) * 4;
-  k_chunk_attn_step<T><<<dim3(s.heads, spans, n_seq), 256, lds, g.stream>>>(s, act, cache, (float*)g_parts.p, seq0, pos);
+template <class T, int NC, int RG, int KI>
+static int run_step_as(const ASpec& s, float* act, T* cache, uint32_t n_seq, uint32_t seq0, uint32_t pos) {
+  const uint32_t parts = cdiv(s.heads / s.kv_heads, RG), n = pos % s.chunk + 1u, unit = 16u * KI;
+  const uint32_t most = std::min<uint32_t>(MAX_SPANS, std::max<uint32_t>(1u, 2u * (uint32_t)g.n_cu / (s.kv_heads * parts * n_seq)));
+  const uint32_t span = cdiv(cdiv(n, std::min(most, cdiv(n, unit))), unit) * unit, spans = cdiv(n, span);
+  if (s.chunk > unit)      // at its full size from the first step on: a graph may be recording when the second span begins
+    if (int r = scratch_need(g_parts, (size_t)n_seq * s.heads * MAX_SPANS * (s.vdim + 2) * 4)) return r;
+  k_chunk_attn_step<T, NC, RG, KI><<<dim3(s.kv_heads * parts, spans, n_seq), 256, 0, g.stream>>>(s, act, cache, (float*)g_parts.p, seq0, pos, span, parts);
   count_launch();
   if (spans > 1) {
     if (int r = check_launch()) return r;
-    k_chunk_attn_join<<<dim3(s.heads, n_seq), 128, 0, g.stream>>>(s, act, (const float*)g_parts.p, spans);
+    k_chunk_attn_join<<<dim3(s.heads, n_seq), 256, 0, g.stream>>>(s, act, (const float*)g_parts.p, spans);
     count_launch();
   }
   return check_launch();
+}
+template <class T>
+static int run_step(const ASpec& s, float* act, T* cache, uint32_t n_seq, uint32_t seq0, uint32_t pos) {
+  const uint32_t rep = s.heads / s.kv_heads;
+  constexpr int KI = sizeof(T) == 2 ? 8 : 4;
+  if (s.dim <= 128u && s.vdim <= 128u)
+    return rep == 1 ? run_step_as<T, 1, 1, KI>(s, act, cache, n_seq, seq0, pos) : rep == 2 ? run_step_as<T, 1, 2, KI>(s, act, cache, n_seq, seq0, pos)
+                                                                                          : run_step_as<T, 1, 4, KI>(s, act, cache, n_seq, seq0, pos);
+  return rep == 1 ? run_step_as<T, 2, 1, KI / 2>(s, act, cache, n_seq, seq0, pos) : run_step_as<T, 2, 2, KI / 2>(s, act, cache, n_seq, seq0, pos);
 }
 
 }  // namespace adamah

@@ -495,21 +495,26 @@ static int row_list(uint32_t h_rows, uint32_t rows, const uint32_t** dev, uint32
 }
 
 // k_merge_norm: dst += scale * sum over the two parts of rms(part) * weight
-__global__ void __launch_bounds__(256)
+template <int NT>
+__global__ void __launch_bounds__(NT)
 k_merge_norm(const AdamahMergeSpec s, float* act) {
-  __shared__ float sh[8];
+  __shared__ float sh[2][NT / 64];
   const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
   const float* a = act + s.a + (uint64_t)blockIdx.x * s.stride;
   const float* b = act + s.b + (uint64_t)blockIdx.x * s.stride;
   float* d = act + s.dst + (uint64_t)blockIdx.x * s.dst_stride;
   float sa = 0.f, sb = 0.f;
-  for (uint32_t i = tid; i < s.dim; i += 256u) { sa = fmaf(a[i], a[i], sa); sb = fmaf(b[i], b[i], sb); }
+#pragma unroll 4
+  for (uint32_t i = tid; i < s.dim; i += NT) { sa = fmaf(a[i], a[i], sa); sb = fmaf(b[i], b[i], sb); }
   sa = wsum64(sa); sb = wsum64(sb);
-  if (lane == 0) { sh[wave] = sa; sh[4 + wave] = sb; }
+  if (lane == 0) { sh[0][wave] = sa; sh[1][wave] = sb; }
   __syncthreads();
-  const float ia = 1.0f / sqrtf(((sh[0] + sh[1]) + (sh[2] + sh[3])) / (float)s.dim + s.eps);
-  const float ib = 1.0f / sqrtf(((sh[4] + sh[5]) + (sh[6] + sh[7])) / (float)s.dim + s.eps);
-  for (uint32_t i = tid; i < s.dim; i += 256u) d[i] += s.scale * (a[i] * ia * act[s.wa + i] + b[i] * ib * act[s.wb + i]);
+  sa = sb = 0.f;
+#pragma unroll
+  for (int w = 0; w < NT / 64; w++) { sa += sh[0][w]; sb += sh[1][w]; }
+  const float ia = 1.0f / sqrtf(sa / (float)s.dim + s.eps), ib = 1.0f / sqrtf(sb / (float)s.dim + s.eps);
+#pragma unroll 4
+  for (uint32_t i = tid; i < s.dim; i += NT) d[i] += s.scale * (a[i] * ia * act[s.wa + i] + b[i] * ib * act[s.wb + i]);
 }
 
 }  // namespace adamah
@@ -558,7 +563,8 @@ int adamah_merge_norm_dev(uint32_t map_act, uint32_t h_spec, uint32_t rows) { AD
   if (!span_ok(s->a, s->stride, rows, s->dim, ma->n_elems) || !span_ok(s->b, s->stride, rows, s->dim, ma->n_elems) ||
       !span_ok(s->dst, s->dst_stride, rows, s->dim, ma->n_elems) || !in_range(s->wa, s->dim, ma->n_elems) ||
       !in_range(s->wb, s->dim, ma->n_elems)) return ADAMAH_ERR_INVALID;
-  k_merge_norm<<<rows, 256, 0, g.stream>>>(*s, (float*)ma->buf);
+  if (rows < 64) k_merge_norm<1024><<<rows, 1024, 0, g.stream>>>(*s, (float*)ma->buf);
+  else k_merge_norm<256><<<rows, 256, 0, g.stream>>>(*s, (float*)ma->buf);
   count_launch();
   return check_launch();
 }

@@ -24,6 +24,7 @@
 namespace adamah {
 
 #define CH 16u            // tokens of a chunk
+#define MAX_TAPS 16       // of the short convolution
 #define VC 32u            // value columns of a decode workgroup
 #define NO_MEMORY 110.0f  // exp(-110) is zero in float32: a stronger decay per token changes nothing, and the sums stay small
 
@@ -48,16 +49,44 @@ __device__ __forceinline__ void block_add3(float& a, float& b, float& c, float* 
   c = (sh[8] + sh[9]) + (sh[10] + sh[11]);
 }
 
-// silu of the causal convolution at token position p for channel ch.  Inputs of this portion: xr (its row, rows
-// x_stride apart, `back` rows of the portion lie before it); older ones: the ring.
-__device__ __forceinline__ float conv_silu(const float* xr, uint32_t x_stride, uint32_t back, const float* ring, uint32_t n_ch,
-                                           uint32_t ch, uint32_t p, const float* w, uint32_t taps) {
-  float a = w[taps - 1u] * xr[ch];
-  for (uint32_t j = 1; j < taps && j <= p; j++) {
-    const float x = j <= back ? *(xr + ((int64_t)ch - (int64_t)((uint64_t)j * x_stride))) : ring[(uint64_t)((p - j) % taps) * n_ch + ch];
-    a = fmaf(w[taps - 1u - j], x, a);
+// silu of the causal convolution at token position p for channel ch, older inputs from the ring only.  The taps' loads do
+// not depend on each other: up to TM of them are asked for at once (TM >= taps).
+template <int TM>
+__device__ __forceinline__ float conv_silu_ring(const float* x, const float* ring, uint32_t n_ch, uint32_t ch, uint32_t p,
+                                                const float* w, uint32_t taps) {
+  float in[TM], wt[TM];
+#pragma unroll
+  for (int j = 0; j < TM; j++) {
+    const bool on = (uint32_t)j < taps && (uint32_t)j <= p;
+    in[j] = !on ? 0.f : j == 0 ? x[ch] : ring[(uint64_t)((p - (uint32_t)j) % taps) * n_ch + ch];
+    wt[j] = on ? w[taps - 1u - (uint32_t)j] : 0.f;
   }
+  float a = 0.f;
+#pragma unroll
+  for (int j = 0; j < TM; j++) a = fmaf(wt[j], in[j], a);
   return silu_f(a);
+}
+// The same for CH consecutive tokens of a portion: rows r0 .. r0 + CH - 1 of x (zero results from row m on), row 0 at
+// position pos; put(t, value).
+template <int TM, class Put>
+__device__ __forceinline__ void conv_silu_rows(const float* x, uint32_t x_stride, uint32_t r0, uint32_t m, const float* ring, uint32_t n_ch,
+                                               uint32_t ch, uint32_t pos, const float* w, uint32_t taps, Put put) {
+  float in[CH + TM - 1], wt[TM];
+#pragma unroll
+  for (int i = 0; i < (int)CH + TM - 1; i++) {
+    const int64_t r = (int64_t)r0 + i - (TM - 1);
+    const bool old = r < 0, on = old ? (uint32_t)-r < taps && (uint32_t)-r <= pos : r < (int64_t)m;
+    in[i] = !on ? 0.f : old ? ring[(uint64_t)((pos + (uint32_t)r) % taps) * n_ch + ch] : x[(uint64_t)r * x_stride + ch];
+  }
+#pragma unroll
+  for (int j = 0; j < TM; j++) wt[j] = (uint32_t)j < taps ? w[taps - 1u - (uint32_t)j] : 0.f;
+#pragma unroll
+  for (int t = 0; t < (int)CH; t++) {
+    float a = 0.f;
+#pragma unroll
+    for (int j = 0; j < TM; j++) a = fmaf(wt[j], in[t + TM - 1 - j], a);
+    put(t, r0 + (uint32_t)t < m ? silu_f(a) : 0.f);
+  }
 }
 
 // dot product of a bf16 matrix row with a float32 vector, by 8 neighbouring lanes (all get the sum)
@@ -78,55 +107,99 @@ __device__ __forceinline__ float dot8(const bf16_t* w, const float* x, uint32_t 
 
 struct LowRank { uint32_t w, k, k_stride, src, src_stride, out, out_stride; };   // what a step needs of a linear spec
 
-// One token of one sequence per blockIdx.z; DN: state rows a thread holds (dim <= 8 DN).
-template <int DN>
+// products of 8-lane rows held in registers: NC 16-byte words of the row per lane
+template <int NC>
+__device__ __forceinline__ float dot8_regs(const uint4 (&w)[NC], const float* x, uint32_t k, uint32_t sub) {
+  float a = 0.f;
+#pragma unroll
+  for (int n = 0; n < NC; n++) {
+    const uint32_t c = sub * 8u + 64u * n, u[4] = {w[n].x, w[n].y, w[n].z, w[n].w};
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      if (c + 2 * i < k) a = fmaf(bf_lo(u[i]), x[c + 2 * i], a);
+      if (c + 2 * i + 1 < k) a = fmaf(bf_hi(u[i]), x[c + 2 * i + 1], a);
+    }
+  }
+  a += __shfl_xor(a, 1, 64); a += __shfl_xor(a, 2, 64); a += __shfl_xor(a, 4, 64);
+  return a;
+}
+
+// One token of one sequence per blockIdx.z; DN: state rows a thread holds (dim <= 8 DN); TM >= taps.  Everything a
+// workgroup reads is asked for at the start: the state, the convolution's inputs, the rows of the low-rank factors (in
+// registers where their rank is at most 128).
+template <int DN, int TM>
 __global__ void __launch_bounds__(256)
 k_delta_step(const DSpec s, const LowRank da, const LowRank ga, float* act, const bf16_t* __restrict__ W, float* state, uint32_t seq0,
              uint32_t pos) {
+  constexpr int NP = DN / 4;                 // decay rows of 8 lanes: 32 a pass
   extern __shared__ float lds[];
   __shared__ float sh[12];
   __shared__ float red[2][8][VC];
   __shared__ float vs[VC];
   const uint32_t D = s.dim, V = s.vdim, tid = threadIdx.x, h = blockIdx.x, v0 = blockIdx.y * VC, row = blockIdx.z;
   float *qs = lds, *ks = qs + D, *gs = ks + D, *lr = gs + D;
-  const uint32_t n_ch = 2u * s.kv_heads * D + s.heads * V, rep = s.heads / s.kv_heads, kv = h / rep;
+  const uint32_t n_ch = 2u * s.kv_heads * D + s.heads * V, rep = s.heads / s.kv_heads, kv = h / rep, sub = tid & 7u;
   const float* x = act + s.x + (uint64_t)row * s.x_stride;
   float* ring = state + (uint64_t)(seq0 + row) * s.seq_stride + s.conv_off;
   float* S = state + (uint64_t)(seq0 + row) * s.seq_stride + s.s_off + (uint64_t)h * D * V;
   const uint32_t qc = kv * D, kc = s.kv_heads * D + kv * D, vc = 2u * s.kv_heads * D + h * V;
   const uint32_t col = tid & 31u, dg = tid >> 5, v = v0 + col;
+  const bool small = da.k_stride <= 128u && ga.k_stride <= 128u;
+  const uint32_t grow = h * V + min(v0 + (tid >> 3), V - 1u);
   float st[DN];
 #pragma unroll
-  for (int i = 0; i < DN; i++) {                       // asked for first: everything below runs under these loads
+  for (int i = 0; i < DN; i++) {
     const uint32_t d = dg + 8u * i;
     st[i] = (pos != 0u && d < D && v < V) ? S[(uint64_t)d * V + v] : 0.f;
+  }
+  uint4 wa[NP][2], wg[2];
+  if (small) {
+#pragma unroll
+    for (int i = 0; i < NP; i++) {
+      const bf16_t* w = W + da.w + (uint64_t)(h * D + min((tid >> 3) + 32u * i, D - 1u)) * da.k_stride;
+#pragma unroll
+      for (int n = 0; n < 2; n++) wa[i][n] = sub * 8u + 64u * n < da.k_stride ? *(const uint4*)(w + sub * 8u + 64u * n) : make_uint4(0, 0, 0, 0);
+    }
+#pragma unroll
+    for (int n = 0; n < 2; n++)
+      wg[n] = sub * 8u + 64u * n < ga.k_stride ? *(const uint4*)(W + ga.w + (uint64_t)grow * ga.k_stride + sub * 8u + 64u * n) : make_uint4(0, 0, 0, 0);
   }
   for (uint32_t i = tid; i < da.k; i += 256u) lr[i] = act[da.src + (uint64_t)row * da.src_stride + i];
   for (uint32_t i = tid; i < ga.k; i += 256u) lr[da.k + i] = act[ga.src + (uint64_t)row * ga.src_stride + i];
   float sq = 0.f, sk = 0.f, qk = 0.f;
-  for (uint32_t d = tid; d < D; d += 256u) {
-    const float a = conv_silu(x, 0, 0, ring, n_ch, qc + d, pos, act + s.cq + (uint64_t)(kv * D + d) * s.taps, s.taps);
-    const float b = conv_silu(x, 0, 0, ring, n_ch, kc + d, pos, act + s.ck + (uint64_t)(kv * D + d) * s.taps, s.taps);
-    qs[d] = a; ks[d] = b;
-    sq = fmaf(a, a, sq); sk = fmaf(b, b, sk); qk = fmaf(a, b, qk);
+  for (uint32_t i = tid; i < 2u * D; i += 256u) {
+    const bool is_k = i >= D;
+    const uint32_t d = is_k ? i - D : i;
+    const float a = conv_silu_ring<TM>(x, ring, n_ch, (is_k ? kc : qc) + d, pos, act + (is_k ? s.ck : s.cq) + (uint64_t)(kv * D + d) * s.taps, s.taps);
+    (is_k ? ks : qs)[d] = a;
+    if (is_k) sk = fmaf(a, a, sk); else sq = fmaf(a, a, sq);
   }
   if (tid < VC && v0 + tid < V)
-    vs[tid] = conv_silu(x, 0, 0, ring, n_ch, vc + v0 + tid, pos, act + s.cv + (uint64_t)(h * V + v0 + tid) * s.taps, s.taps);
-  block_add3(sq, sk, qk, sh);
+    vs[tid] = conv_silu_ring<TM>(x, ring, n_ch, vc + v0 + tid, pos, act + s.cv + (uint64_t)(h * V + v0 + tid) * s.taps, s.taps);
+  const float ea = expf(act[s.a_log + h]), beta = sigmoid_f(x[s.x_b + h]);
+  __syncthreads();
+  for (uint32_t d = tid; d < D; d += 256u) qk = fmaf(qs[d], ks[d], qk);
+  if (small) {
+#pragma unroll
+    for (int i = 0; i < NP; i++) {
+      const uint32_t d = (tid >> 3) + 32u * i;
+      const float a = dot8_regs<2>(wa[i], lr, da.k, sub);
+      if (sub == 0 && d < D) gs[d] = expf(-ea * softplus_f(a + act[s.dt_bias + h * D + d]));
+    }
+    const float a = dot8_regs<2>(wg, lr + da.k, ga.k, sub);
+    if (sub == 0 && v0 + (tid >> 3) < V) act[ga.out + (uint64_t)row * ga.out_stride + grow] = a;
+  } else {
+    for (uint32_t d = tid >> 3; d < ((D + 31u) & ~31u); d += 32u) {      // whole waves take part in the dot products
+      const uint32_t r = h * D + min(d, D - 1u);
+      const float a = dot8(W + da.w + (uint64_t)r * da.k_stride, lr, da.k, da.k_stride, sub);
+      if (sub == 0 && d < D) gs[d] = expf(-ea * softplus_f(a + act[s.dt_bias + r]));
+    }
+    const float a = dot8(W + ga.w + (uint64_t)grow * ga.k_stride, lr + da.k, ga.k, ga.k_stride, sub);
+    if (sub == 0 && v0 + (tid >> 3) < V) act[ga.out + (uint64_t)row * ga.out_stride + grow] = a;
+  }
+  block_add3(sq, sk, qk, sh);                  // (its barriers also publish gs)
   const float iq = 1.0f / sqrtf(sq + 1e-6f) / sqrtf((float)D), ik = 1.0f / sqrtf(sk + 1e-6f);
   qk = qk * iq * ik;
-  const float ea = expf(act[s.a_log + h]);
-  for (uint32_t d = tid >> 3; d < ((D + 31u) & ~31u); d += 32u) {      // whole waves take part in the dot products
-    const uint32_t r = h * D + min(d, D - 1u);
-    const float a = dot8(W + da.w + (uint64_t)r * da.k_stride, lr, da.k, da.k_stride, tid & 7u);
-    if ((tid & 7u) == 0 && d < D) gs[d] = expf(-ea * softplus_f(a + act[s.dt_bias + r]));
-  }
-  {
-    const uint32_t d = tid >> 3, r = h * V + min(v0 + d, V - 1u);
-    const float a = dot8(W + ga.w + (uint64_t)r * ga.k_stride, lr + da.k, ga.k, ga.k_stride, tid & 7u);
-    if ((tid & 7u) == 0 && v0 + d < V) act[ga.out + (uint64_t)row * ga.out_stride + r] = a;
-  }
-  __syncthreads();
   float pk = 0.f, pq = 0.f;
 #pragma unroll
   for (int i = 0; i < DN; i++) {
@@ -142,7 +215,6 @@ k_delta_step(const DSpec s, const LowRank da, const LowRank ga, float* act, cons
 #pragma unroll
   for (int i = 0; i < 8; i++) { pk += red[0][i][col]; pq += red[1][i][col]; }
   if (v < V) {
-    const float beta = sigmoid_f(x[s.x_b + h]);
     const float u = beta * (vs[col] - pk * ik);
     if (dg == 0) act[s.out + (uint64_t)row * s.out_stride + h * V + v] = fmaf(u, qk, pq * iq);
     const float uk = u * ik;
@@ -218,61 +290,72 @@ k_retention_step(const RSpec s, float* act, float* state, uint32_t seq0, uint32_
 struct ChunkDims { uint32_t Dp, Vp, n_chunks; };
 __host__ __device__ inline uint32_t chunk_floats(uint32_t Dp, uint32_t Vp) { return 49u * Dp + 256u + 16u * Vp; }
 
+// Columns of q and k (a thread each) run through their convolution in registers, then those of v and of the decay.
+template <int TM>
 __global__ void __launch_bounds__(256)
 k_delta_prep(const DSpec s, uint32_t dec_out, uint32_t dec_stride, const float* __restrict__ act, const float* __restrict__ state,
              float* __restrict__ scratch, ChunkDims cd, uint32_t m, uint32_t seq0, uint32_t pos) {
   extern __shared__ float lds[];
-  __shared__ float A[CH][CH + 1], M[CH][CH + 1], beta[CH];
+  __shared__ __attribute__((aligned(16))) float A[CH][CH + 4], M[CH][CH + 4];
+  __shared__ float beta[CH], iq[CH], ik[CH];
   const uint32_t D = s.dim, V = s.vdim, tid = threadIdx.x, c0 = blockIdx.x * CH, h = blockIdx.y, P = D + 1u;
-  float *qs = lds, *ks = qs + CH * P, *G = ks + CH * P;
+  float *qs = lds, *ks = qs + CH * P, *G = ks + CH * P, *vs = G + CH * P;             // G: log2 of the running decay; vs [CH][Vp]
   const uint32_t n_ch = 2u * s.kv_heads * D + s.heads * V, kv = h / (s.heads / s.kv_heads);
   const uint32_t qc = kv * D, kc = s.kv_heads * D + kv * D, vc = 2u * s.kv_heads * D + h * V;
   const float* x = act + s.x;
   const float* ring = state + (uint64_t)seq0 * s.seq_stride + s.conv_off;
   float* out = scratch + ((uint64_t)h * cd.n_chunks + blockIdx.x) * chunk_floats(cd.Dp, cd.Vp);
   float *oW = out, *oQ = oW + CH * cd.Dp, *oK = oQ + CH * cd.Dp, *oB = oK + CH * cd.Dp, *oU = oB + 256u, *oG = oU + CH * cd.Vp;
-  for (uint32_t i = tid; i < CH * D; i += 256u) {
-    const uint32_t t = i / D, d = i - t * D, r = c0 + t;
-    float a = 0.f, b = 0.f;
-    if (r < m) {
-      const float* xr = x + (uint64_t)r * s.x_stride;
-      a = conv_silu(xr, s.x_stride, r, ring, n_ch, qc + d, pos + r, act + s.cq + (uint64_t)(kv * D + d) * s.taps, s.taps);
-      b = conv_silu(xr, s.x_stride, r, ring, n_ch, kc + d, pos + r, act + s.ck + (uint64_t)(kv * D + d) * s.taps, s.taps);
-    }
-    qs[t * P + d] = a; ks[t * P + d] = b;
+  for (uint32_t i = tid; i < 2u * D; i += 256u) {
+    const bool is_k = i >= D;
+    const uint32_t d = is_k ? i - D : i;
+    float* to = (is_k ? ks : qs) + d;
+    conv_silu_rows<TM>(x, s.x_stride, c0, m, ring, n_ch, (is_k ? kc : qc) + d, pos, act + (is_k ? s.ck : s.cq) + (uint64_t)(kv * D + d) * s.taps,
+                       s.taps, [&](int t, float v) { to[t * P] = v; });
   }
   if (tid < CH) beta[tid] = c0 + tid < m ? sigmoid_f(x[(uint64_t)(c0 + tid) * s.x_stride + s.x_b + h]) : 0.f;
   const float ea = expf(act[s.a_log + h]);
-  for (uint32_t d = tid; d < D; d += 256u) {                 // running logarithms of the decay
-    const float bias = act[s.dt_bias + h * D + d];
-    float lg = 0.f;
-    for (uint32_t t = 0; t < CH; t++) {
-      if (c0 + t < m) lg -= fminf(ea * softplus_f(act[dec_out + (uint64_t)(c0 + t) * dec_stride + h * D + d] + bias), NO_MEMORY);
-      G[t * P + d] = lg;
+  const uint32_t v_items = (V + 63u) & ~63u;                 // whole waves do one or the other
+  for (uint32_t i = tid; i < v_items + D; i += 256u) {
+    if (i < v_items) {
+      if (i < V) conv_silu_rows<TM>(x, s.x_stride, c0, m, ring, n_ch, vc + i, pos, act + s.cv + (uint64_t)(h * V + i) * s.taps, s.taps,
+                                    [&](int t, float v) { vs[t * cd.Vp + i] = v; });
+    } else {
+      const uint32_t d = i - v_items;
+      const float bias = act[s.dt_bias + h * D + d];
+      float z[CH];
+#pragma unroll
+      for (int t = 0; t < (int)CH; t++) z[t] = c0 + t < m ? act[dec_out + (uint64_t)(c0 + t) * dec_stride + h * D + d] + bias : 0.f;
+      float lg = 0.f;
+#pragma unroll
+      for (int t = 0; t < (int)CH; t++) {
+        if (c0 + t < m) lg -= fminf(ea * softplus_f(z[t]), NO_MEMORY) * 1.44269504f;
+        G[t * P + d] = lg;
+      }
     }
   }
   __syncthreads();
-  {                                                          // unit q and k: 8 threads a row, 32 rows
+  {                                                          // lengths of q and k: 8 threads a row, 32 rows
     const uint32_t rr = tid >> 3, sub = tid & 7u;
-    float* v = (rr < CH ? qs : ks) + (rr & (CH - 1u)) * P;
+    const float* v = (rr < CH ? qs : ks) + (rr & (CH - 1u)) * P;
     float ss = 0.f;
     for (uint32_t d = sub; d < D; d += 8u) ss = fmaf(v[d], v[d], ss);
     ss += __shfl_xor(ss, 1, 64); ss += __shfl_xor(ss, 2, 64); ss += __shfl_xor(ss, 4, 64);
-    const float inv = 1.0f / sqrtf(ss + 1e-6f) / (rr < CH ? sqrtf((float)D) : 1.0f);
-    for (uint32_t d = sub; d < D; d += 8u) v[d] *= inv;
+    if (sub == 0) (rr < CH ? iq : ik)[rr & (CH - 1u)] = 1.0f / sqrtf(ss + 1e-6f) / (rr < CH ? sqrtf((float)D) : 1.0f);
   }
   __syncthreads();
   {
     const uint32_t t = tid >> 4, r = tid & 15u;
     float a = 0.f, b = 0.f;
     if (r <= t) {
+#pragma unroll 4
       for (uint32_t d = 0; d < D; d++) {
-        const float e = expf(G[t * P + d] - G[r * P + d]) * ks[r * P + d];
+        const float e = __builtin_amdgcn_exp2f(G[t * P + d] - G[r * P + d]) * ks[r * P + d];
         a = fmaf(ks[t * P + d], e, a); b = fmaf(qs[t * P + d], e, b);
       }
     }
-    A[t][r] = r < t ? a : 0.f;
-    oB[t * 16u + r] = b;
+    A[t][r] = r < t ? a * ik[t] * ik[r] * beta[t] : 0.f;
+    oB[t * 16u + r] = b * iq[t] * ik[r];
   }
   __syncthreads();
   if (tid < CH) {                                            // column tid of the inverse, forward substitution
@@ -281,46 +364,43 @@ k_delta_prep(const DSpec s, uint32_t dec_out, uint32_t dec_stride, const float* 
     for (int t = 0; t < (int)CH; t++) {
       float a = (uint32_t)t == tid ? 1.f : 0.f;
 #pragma unroll
-      for (int r = 0; r < t; r++) a = fmaf(-beta[t] * A[t][r], y[r], a);
+      for (int r = 0; r < t; r++) a = fmaf(-A[t][r], y[r], a);
       y[t] = a;
       M[t][tid] = a * beta[tid];
     }
   }
   __syncthreads();
-  for (uint32_t d = tid; d < cd.Dp; d += 256u) {
-    float kg[CH];
-    const float gl = d < D ? G[15u * P + d] : 0.f;
+  for (uint32_t i = tid; i < 2u * cd.Dp + cd.Vp; i += 256u) {
+    if (i < cd.Dp) {
+      const uint32_t d = i;
+      const bool in = d < D;
+      const float gl = in ? G[15u * P + d] : 0.f;
+      float kt[CH];
 #pragma unroll
-    for (int t = 0; t < (int)CH; t++) {
-      const float lg = d < D ? G[t * P + d] : 0.f, k = d < D ? ks[t * P + d] : 0.f, q = d < D ? qs[t * P + d] : 0.f;
-      const float e = expf(lg);
-      kg[t] = k * e;
-      oQ[t * cd.Dp + d] = q * e;
-      oK[d * 16u + t] = k * expf(gl - lg);
-    }
-    oG[d] = expf(gl);
+      for (int t = 0; t < (int)CH; t++) {
+        const float lg = in ? G[t * P + d] : 0.f;
+        oQ[t * cd.Dp + d] = in ? qs[t * P + d] * iq[t] * __builtin_amdgcn_exp2f(lg) : 0.f;
+        kt[t] = in ? ks[t * P + d] * ik[t] * __builtin_amdgcn_exp2f(gl - lg) : 0.f;
+      }
 #pragma unroll
-    for (int t = 0; t < (int)CH; t++) {
-      float a = 0.f;
+      for (int t = 0; t < (int)CH; t += 4) *(f4_t*)(oK + d * 16u + t) = (f4_t){kt[t], kt[t + 1], kt[t + 2], kt[t + 3]};
+      oG[d] = __builtin_amdgcn_exp2f(gl);
+    } else {
+      const bool is_u = i >= 2u * cd.Dp;
+      const uint32_t d = is_u ? i - 2u * cd.Dp : i - cd.Dp;
+      float y[CH];
 #pragma unroll
-      for (int r = 0; r <= t; r++) a = fmaf(M[t][r], kg[r], a);
-      oW[t * cd.Dp + d] = a;
-    }
-  }
-  for (uint32_t v = tid; v < cd.Vp; v += 256u) {
-    float y[CH];
+      for (int t = 0; t < (int)CH; t++)
+        y[t] = is_u ? (d < V ? vs[t * cd.Vp + d] : 0.f) : d < D ? ks[t * P + d] * ik[t] * __builtin_amdgcn_exp2f(G[t * P + d]) : 0.f;
+      float* o = is_u ? oU + d : oW + d;
+      const uint32_t os = is_u ? cd.Vp : cd.Dp;
 #pragma unroll
-    for (int t = 0; t < (int)CH; t++) {
-      const uint32_t r = c0 + t;
-      y[t] = (r < m && v < V) ? conv_silu(x + (uint64_t)r * s.x_stride, s.x_stride, r, ring, n_ch, vc + v, pos + r,
-                                          act + s.cv + (uint64_t)(h * V + v) * s.taps, s.taps) : 0.f;
-    }
+      for (int t = 0; t < (int)CH; t++) {
+        float a = 0.f;
 #pragma unroll
-    for (int t = 0; t < (int)CH; t++) {
-      float a = 0.f;
-#pragma unroll
-      for (int r = 0; r <= t; r++) a = fmaf(M[t][r], y[r], a);
-      oU[t * cd.Vp + v] = a;
+        for (int r = 0; r <= t; r++) a = fmaf(M[t][r], y[r], a);
+        o[t * os] = a;
+      }
     }
   }
 }
@@ -329,9 +409,9 @@ __global__ void __launch_bounds__(256)
 k_retention_prep(const RSpec s, const float* __restrict__ act, float* __restrict__ scratch, ChunkDims cd, uint32_t m, uint32_t pos) {
   extern __shared__ float lds[];
   __shared__ float pw[CH + 1];
-  const uint32_t D = s.dim, V = s.vdim, tid = threadIdx.x, c0 = blockIdx.x * CH, h = blockIdx.y, P = D + 1u;
+  const uint32_t D = s.dim, V = s.vdim, tid = threadIdx.x, c0 = blockIdx.x * CH, h = blockIdx.y, P = D + 1u, half = s.rot_dims >> 1;
   const uint32_t L = min(CH, m - c0);
-  float *qs = lds, *ks = qs + CH * P;
+  float *qs = lds, *ks = qs + CH * P, *cs = ks + CH * P, *sn = cs + CH * half;
   float* out = scratch + ((uint64_t)h * cd.n_chunks + blockIdx.x) * chunk_floats(cd.Dp, cd.Vp);
   float *oQ = out + CH * cd.Dp, *oK = oQ + CH * cd.Dp, *oB = oK + CH * cd.Dp, *oU = oB + 256u, *oG = oU + CH * cd.Vp;
   const float kscale = 1.0f / sqrtf((float)D);
@@ -340,33 +420,60 @@ k_retention_prep(const RSpec s, const float* __restrict__ act, float* __restrict
     pw[0] = 1.f;
     for (uint32_t i = 1; i <= CH; i++) pw[i] = pw[i - 1] * dec;
   }
-  for (uint32_t i = tid; i < CH * D; i += 256u) {
-    const uint32_t t = i / D, d = i - t * D, r = c0 + t;
-    const float* xr = act + s.x + (uint64_t)r * s.x_stride;
-    qs[t * P + d] = r < m ? rotated(xr + s.x_q + h * D, act + s.freq, d, s.rot_dims, pos + r) : 0.f;
-    ks[t * P + d] = r < m ? rotated(xr + s.x_k + h * D, act + s.freq, d, s.rot_dims, pos + r) * kscale : 0.f;
+  for (uint32_t i = tid; i < 2u * D; i += 256u) {
+    const bool is_k = i >= D;
+    const uint32_t d = is_k ? i - D : i;
+    const float* src = act + s.x + (is_k ? s.x_k : s.x_q) + h * D + d;
+    float* to = (is_k ? ks : qs) + d;
+    float v[CH];
+#pragma unroll
+    for (int t = 0; t < (int)CH; t++) v[t] = c0 + t < m ? src[(uint64_t)(c0 + t) * s.x_stride] : 0.f;
+#pragma unroll
+    for (int t = 0; t < (int)CH; t++) to[t * P] = is_k ? v[t] * kscale : v[t];
+  }
+  for (uint32_t i = tid; i < CH * half; i += 256u) {
+    const uint32_t t = i / half, d = i - t * half;
+    float a, b;
+    sincosf((float)(pos + c0 + t) * act[s.freq + d], &a, &b);
+    sn[i] = a; cs[i] = b;
+  }
+  for (uint32_t v = tid; v < cd.Vp; v += 256u) {
+    float y[CH];
+#pragma unroll
+    for (int t = 0; t < (int)CH; t++) y[t] = (c0 + t < m && v < V) ? act[s.x + (uint64_t)(c0 + t) * s.x_stride + s.x_v + h * V + v] : 0.f;
+#pragma unroll
+    for (int t = 0; t < (int)CH; t++) oU[t * cd.Vp + v] = y[t];
+  }
+  __syncthreads();
+  for (uint32_t i = tid; i < 2u * CH * half; i += 256u) {     // turn the pairs in place
+    const bool is_k = i >= CH * half;
+    const uint32_t j = is_k ? i - CH * half : i, t = j / half, d = j - t * half;
+    float* r = (is_k ? ks : qs) + t * P;
+    const float a = r[d], b = r[d + half];
+    r[d] = a * cs[j] - b * sn[j];
+    r[d + half] = b * cs[j] + a * sn[j];
   }
   __syncthreads();
   {
     const uint32_t t = tid >> 4, r = tid & 15u;
     float b = 0.f;
     if (r <= t) {
+#pragma unroll 4
       for (uint32_t d = 0; d < D; d++) b = fmaf(qs[t * P + d], ks[r * P + d], b);
       b *= pw[t - r];
     }
     oB[t * 16u + r] = b;
   }
   for (uint32_t d = tid; d < cd.Dp; d += 256u) {
+    float kt[CH];
 #pragma unroll
     for (int t = 0; t < (int)CH; t++) {
       oQ[t * cd.Dp + d] = d < D ? qs[t * P + d] * pw[t + 1] : 0.f;
-      oK[d * 16u + t] = (d < D && (uint32_t)t < L) ? ks[t * P + d] * pw[L - 1u - (uint32_t)t] : 0.f;
+      kt[t] = (d < D && (uint32_t)t < L) ? ks[t * P + d] * pw[L - 1u - min((uint32_t)t, L - 1u)] : 0.f;
     }
+#pragma unroll
+    for (int t = 0; t < (int)CH; t += 4) *(f4_t*)(oK + d * 16u + t) = (f4_t){kt[t], kt[t + 1], kt[t + 2], kt[t + 3]};
     oG[d] = pw[L];
-  }
-  for (uint32_t i = tid; i < CH * cd.Vp; i += 256u) {
-    const uint32_t t = i / cd.Vp, v = i - t * cd.Vp, r = c0 + t;
-    oU[i] = (r < m && v < V) ? act[s.x + (uint64_t)r * s.x_stride + s.x_v + h * V + v] : 0.f;
   }
 }
 
@@ -513,7 +620,7 @@ int adamah_delta_rule_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, 
   if (!ma || !mw || mw->dtype != DTYPE_BF16 || !s || !da || !ga || n_seq == 0 || rows == 0 || (n_seq > 1 && rows > 1)) return ADAMAH_ERR_INVALID;
   Map* ms = get_f32_map(s->state_map);
   const uint64_t D = s->dim, V = s->vdim, H = s->heads, KH = s->kv_heads, n_tok = (uint64_t)n_seq * rows;
-  if (!ms || D == 0 || D > 256 || V == 0 || H == 0 || KH == 0 || H % KH || s->taps == 0) return ADAMAH_ERR_INVALID;
+  if (!ms || D == 0 || D > 256 || V == 0 || H == 0 || KH == 0 || H % KH || s->taps == 0 || s->taps > MAX_TAPS) return ADAMAH_ERR_INVALID;
   const uint64_t n_ch = 2 * KH * D + H * V;
   if (s->x_stride < n_ch || s->x_b + H > s->x_stride) return ADAMAH_ERR_INVALID;
   if (!rows_ok(s->x, s->x_stride, n_tok, s->x_stride, ma->n_elems) || !rows_ok(s->out, s->out_stride, n_tok, H * V, ma->n_elems)) return ADAMAH_ERR_INVALID;
@@ -533,9 +640,10 @@ int adamah_delta_rule_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, 
     if (lds > 48000) return ADAMAH_ERR_INVALID;
     const dim3 grid((uint32_t)H, cdiv(V, VC), n_seq);
     const bf16_t* W = (const bf16_t*)mw->buf;
-    if (D <= 64) k_delta_step<8><<<grid, 256, lds, g.stream>>>(*s, low_rank(*da), low_rank(*ga), act, W, state, seq0, pos);
-    else if (D <= 128) k_delta_step<16><<<grid, 256, lds, g.stream>>>(*s, low_rank(*da), low_rank(*ga), act, W, state, seq0, pos);
-    else k_delta_step<32><<<grid, 256, lds, g.stream>>>(*s, low_rank(*da), low_rank(*ga), act, W, state, seq0, pos);
+#define STEP(DN, TM) k_delta_step<DN, TM><<<grid, 256, lds, g.stream>>>(*s, low_rank(*da), low_rank(*ga), act, W, state, seq0, pos)
+    if (s->taps <= 4) { if (D <= 64) STEP(8, 4); else if (D <= 128) STEP(16, 4); else STEP(32, 4); }
+    else { if (D <= 64) STEP(8, MAX_TAPS); else if (D <= 128) STEP(16, MAX_TAPS); else STEP(32, MAX_TAPS); }
+#undef STEP
     count_launch();
     return check_launch();
   }
@@ -543,8 +651,16 @@ int adamah_delta_rule_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, 
   if (int r = adamah_linear_dev(map_act, map_opnd, map_wt, h_gate, 0, rows)) return r;
   const ChunkDims cd = {(uint32_t)((D + 63) / 64 * 64), (uint32_t)((V + 15) / 16 * 16), cdiv(rows, CH)};
   if (int r = scratch_need(g_chunks, (size_t)H * cd.n_chunks * chunk_floats(cd.Dp, cd.Vp) * 4)) return r;
-  const size_t lds = (size_t)3 * CH * (D + 1) * 4;
-  k_delta_prep<<<dim3(cd.n_chunks, (uint32_t)H), 256, lds, g.stream>>>(*s, da->out, da->out_stride, act, state, (float*)g_chunks.p, cd, rows, seq0, pos);
+  const size_t lds = (size_t)CH * (3 * (D + 1) + cd.Vp) * 4;
+  if (lds > 120000) return ADAMAH_ERR_INVALID;
+#define PREP(TM)                                                                                                                      \
+  do {                                                                                                                                \
+    if (lds > 60000) hipFuncSetAttribute((const void*)k_delta_prep<TM>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);         \
+    k_delta_prep<TM><<<dim3(cd.n_chunks, (uint32_t)H), 256, lds, g.stream>>>(*s, da->out, da->out_stride, act, state,                 \
+                                                                            (float*)g_chunks.p, cd, rows, seq0, pos);                \
+  } while (0)
+  if (s->taps <= 4) PREP(4); else PREP(MAX_TAPS);
+#undef PREP
   count_launch();
   if (int r = check_launch()) return r;
   ScanArgs a = {s->heads, s->dim, s->vdim, s->out, s->out_stride, s->s_off, rows, pos, cd, s->kv_heads, s->taps, s->conv_off, s->x, s->x_stride};
@@ -575,7 +691,7 @@ int adamah_retention_dev(uint32_t map_act, uint32_t h_spec, uint32_t n_seq, uint
   }
   const ChunkDims cd = {(uint32_t)((D + 63) / 64 * 64), (uint32_t)((V + 15) / 16 * 16), cdiv(rows, CH)};
   if (int r = scratch_need(g_chunks, (size_t)H * cd.n_chunks * chunk_floats(cd.Dp, cd.Vp) * 4)) return r;
-  k_retention_prep<<<dim3(cd.n_chunks, (uint32_t)H), 256, (size_t)2 * CH * (D + 1) * 4, g.stream>>>(*s, act, (float*)g_chunks.p, cd, rows, pos);
+  k_retention_prep<<<dim3(cd.n_chunks, (uint32_t)H), 256, (size_t)CH * (2 * (D + 1) + s->rot_dims) * 4, g.stream>>>(*s, act, (float*)g_chunks.p, cd, rows, pos);
   count_launch();
   if (int r = check_launch()) return r;
   ScanArgs a = {s->heads, s->dim, s->vdim, s->out, s->out_stride, s->s_off, rows, pos, cd, 0, 0, 0, 0, 0};
