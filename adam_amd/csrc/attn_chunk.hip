@@ -20,6 +20,8 @@ namespace adamah {
 
 typedef AdamahChunkAttnSpec ASpec;
 #define MAX_SPANS 64u
+#define STEP_WAVES 8u     // of a workgroup that decodes one token
+#define LOG2E 1.44269504f
 #define ATT_MASKED (-1.0e30f)
 
 __device__ __forceinline__ float wsumf(float v) {
@@ -55,12 +57,12 @@ template <> struct Eight<bf16_t> {
 // ---- one token ------------------------------------------------------------------------------------------------------
 // grid (key heads * groups of RG query heads, spans, sequences).  Sixteen lanes share a key: lane l16 holds columns
 // 8 l16 + 128 c; a wave takes 4 KI keys at a time, their keys and values asked for together.  part: per (sequence, head,
-// span) vdim + 2 floats {max, sum, values}, used when there is more than one span.
+// span) vdim + 2 floats {max in powers of two, sum, values}, used when there is more than one span.
 template <class T, int NC, int RG, int KI>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(STEP_WAVES * 64)
 k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq0, uint32_t pos, uint32_t span, uint32_t parts) {
   __shared__ float qb[RG][128 * NC];
-  __shared__ float ob[4][RG][128 * NC], ml[4][RG][2];
+  __shared__ float ob[STEP_WAVES][RG][128 * NC], ml[STEP_WAVES][RG][2];
   const uint32_t D = s.dim, V = s.vdim, D8 = (D + 7u) & ~7u, V8 = (V + 7u) & ~7u, tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
   const uint32_t row = blockIdx.z, rep = s.heads / s.kv_heads, kv = blockIdx.x / parts, h0 = kv * rep + (blockIdx.x - kv * parts) * RG;
   const uint32_t nh = min((uint32_t)RG, (kv + 1u) * rep - h0);       // query heads of this workgroup
@@ -71,14 +73,31 @@ k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq
   T* K = cache + (uint64_t)(seq0 + row) * s.seq_stride + s.k_off + (uint64_t)kv * s.chunk * D8;
   T* Vc = cache + (uint64_t)(seq0 + row) * s.seq_stride + s.v_off + (uint64_t)kv * s.chunk * V8;
   const bool own = k1 == n;                                     // this span ends with the token itself
+  Eight<T> kr[KI][NC], vr[KI][NC];
+  auto fetch = [&](uint32_t kb) {
+#pragma unroll
+    for (int j = 0; j < KI; j++) {
+      const uint32_t key = kb + kq + 4u * j;
+#pragma unroll
+      for (int c = 0; c < NC; c++) {
+        const uint32_t d = l16 * 8u + 128u * c;
+        kr[j][c].zero(); vr[j][c].zero();
+        if (key + 1u < n && key < k1) {
+          if (d < D8) kr[j][c].load(K + (uint64_t)key * D8 + d);
+          if (d < V8) vr[j][c].load(Vc + (uint64_t)key * V8 + d);
+        }
+      }
+    }
+  };
+  fetch(k0 + wave * 4u * KI);                                   // the first keys are on their way while the queries are staged
   float iv = 0.f;
   if (own) {
     for (uint32_t d = lane; d < V; d += 64u) iv = fmaf(xv[d], xv[d], iv);
     iv = 1.0f / sqrtf(wsumf(iv) / (float)V + s.eps);
   }
-  for (uint32_t i = tid; i < RG * 128u * NC; i += 256u) {
+  for (uint32_t i = tid; i < RG * 128u * NC; i += STEP_WAVES * 64u) {
     const uint32_t r = i / (128u * NC), d = i - r * (128u * NC);
-    qb[r][d] = (r < nh && d < D) ? x[s.x_q + (h0 + r) * D + d] * s.scale : 0.f;
+    qb[r][d] = (r < nh && d < D) ? x[s.x_q + (h0 + r) * D + d] * (s.scale * LOG2E) : 0.f;
   }
   float r1[RG], r2[RG], mx[RG], sum[RG], o[RG][NC][8];
 #pragma unroll
@@ -92,26 +111,27 @@ k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq
       for (int i = 0; i < 8; i++) o[r][c][i] = 0.f;
   }
   __syncthreads();
-  for (uint32_t kb = k0 + wave * 4u * KI; kb < k1; kb += 16u * KI) {
-    Eight<T> kr[KI][NC], vr[KI][NC];
+  for (uint32_t kb = k0 + wave * 4u * KI; kb < k1; kb += STEP_WAVES * 4u * KI) {
+    if (kb >= k0 + STEP_WAVES * 4u * KI) fetch(kb);
+    if (own && n - 1u - kb < 4u * KI) {                         // the token's own key and value
 #pragma unroll
-    for (int j = 0; j < KI; j++) {
-      const uint32_t key = kb + kq + 4u * j;
+      for (int j = 0; j < KI; j++)
+        if (kb + kq + 4u * j + 1u == n) {
 #pragma unroll
-      for (int c = 0; c < NC; c++) {
-        const uint32_t d = l16 * 8u + 128u * c;
-        kr[j][c].zero(); vr[j][c].zero();
-        if (key + 1u < n && key < k1) {
-          if (d < D8) kr[j][c].load(K + (uint64_t)key * D8 + d);
-          if (d < V8) vr[j][c].load(Vc + (uint64_t)key * V8 + d);
-        } else if (key + 1u == n) {
-          float a[8], b[8];
+          for (int c = 0; c < NC; c++) {
+            const uint32_t d = l16 * 8u + 128u * c;
+            float a[8], b[8];
 #pragma unroll
-          for (int i = 0; i < 8; i++) { a[i] = d + i < D ? xk[d + i] : 0.f; b[i] = d + i < V ? xv[d + i] * iv : 0.f; }
-          kr[j][c].set(a); vr[j][c].set(b);
+            for (int i = 0; i < 8; i++) { a[i] = d + i < D ? xk[d + i] : 0.f; b[i] = d + i < V ? xv[d + i] * iv : 0.f; }
+            kr[j][c].set(a); vr[j][c].set(b);
+          }
         }
-      }
     }
+    float kk[KI][NC][8], vv[KI][NC][8];
+#pragma unroll
+    for (int j = 0; j < KI; j++)
+#pragma unroll
+      for (int c = 0; c < NC; c++) { kr[j][c].get(kk[j][c]); vr[j][c].get(vv[j][c]); }
 #pragma unroll
     for (int r = 0; r < RG; r++) {
       float sc[KI], top = ATT_MASKED;
@@ -123,23 +143,19 @@ k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq
 #pragma unroll
         for (int i = 0; i < 8; i++) q[i] = qb[r][128u * c + l16 * 8u + i];
 #pragma unroll
-        for (int j = 0; j < KI; j++) {
-          float kk[8];
-          kr[j][c].get(kk);
+        for (int j = 0; j < KI; j++)
 #pragma unroll
-          for (int i = 0; i < 8; i++) sc[j] = fmaf(kk[i], q[i], sc[j]);
-        }
+          for (int i = 0; i < 8; i++) sc[j] = fmaf(kk[j][c][i], q[i], sc[j]);
       }
 #pragma unroll
       for (int j = 0; j < KI; j++) {
-        float a = sc[j];
-        a += __shfl_xor(a, 1, 64); a += __shfl_xor(a, 2, 64); a += __shfl_xor(a, 4, 64); a += __shfl_xor(a, 8, 64);
+        const float a = row16_sum(sc[j]);
         const uint32_t key = kb + kq + 4u * j;
-        sc[j] = key < k1 ? a - r1[r] * logf(fmaf(r2[r], (float)(n - 1u - key), 1.0f)) : ATT_MASKED;
+        sc[j] = key < k1 ? a - r1[r] * __builtin_amdgcn_logf(fmaf(r2[r], (float)(n - 1u - key), 1.0f)) : ATT_MASKED;
         top = fmaxf(top, sc[j]);
       }
       top = fmaxf(top, __shfl_xor(top, 16, 64)); top = fmaxf(top, __shfl_xor(top, 32, 64));
-      const float nm = fmaxf(mx[r], top), al = expf(mx[r] - nm);
+      const float nm = fmaxf(mx[r], top), al = __builtin_amdgcn_exp2f(mx[r] - nm);
       mx[r] = nm;
       sum[r] *= al;
 #pragma unroll
@@ -148,15 +164,12 @@ k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq
         for (int i = 0; i < 8; i++) o[r][c][i] *= al;
 #pragma unroll
       for (int j = 0; j < KI; j++) {
-        const float p = sc[j] > 0.5f * ATT_MASKED ? expf(sc[j] - nm) : 0.f;
+        const float p = sc[j] > 0.5f * ATT_MASKED ? __builtin_amdgcn_exp2f(sc[j] - nm) : 0.f;
         sum[r] += p;
 #pragma unroll
-        for (int c = 0; c < NC; c++) {
-          float vv[8];
-          vr[j][c].get(vv);
+        for (int c = 0; c < NC; c++)
 #pragma unroll
-          for (int i = 0; i < 8; i++) o[r][c][i] = fmaf(p, vv[i], o[r][c][i]);
-        }
+          for (int i = 0; i < 8; i++) o[r][c][i] = fmaf(p, vv[j][c][i], o[r][c][i]);
       }
     }
   }
@@ -174,12 +187,14 @@ k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq
       }
   }
   __syncthreads();
-  for (uint32_t i = tid; i < nh * V; i += 256u) {
+  for (uint32_t i = tid; i < nh * V; i += STEP_WAVES * 64u) {
     const uint32_t r = i / V, d = i - r * V, h = h0 + r;
-    const float m4 = fmaxf(fmaxf(ml[0][r][0], ml[1][r][0]), fmaxf(ml[2][r][0], ml[3][r][0]));
+    float m4 = ml[0][r][0];
+#pragma unroll
+    for (uint32_t w = 1; w < STEP_WAVES; w++) m4 = fmaxf(m4, ml[w][r][0]);
     float a = 0.f, t = 0.f;
 #pragma unroll
-    for (int w = 0; w < 4; w++) { const float e = expf(ml[w][r][0] - m4); a = fmaf(e, ob[w][r][d], a); t = fmaf(e, ml[w][r][1], t); }
+    for (uint32_t w = 0; w < STEP_WAVES; w++) { const float e = __builtin_amdgcn_exp2f(ml[w][r][0] - m4); a = fmaf(e, ob[w][r][d], a); t = fmaf(e, ml[w][r][1], t); }
     if (gridDim.y == 1) act[s.out + (uint64_t)row * s.out_stride + h * V + d] = a / t;
     else {
       float* p = part + (((uint64_t)row * s.heads + h) * gridDim.y + blockIdx.y) * (V + 2u);
@@ -188,8 +203,8 @@ k_chunk_attn_step(const ASpec s, float* act, T* cache, float* part, uint32_t seq
     }
   }
   if (own && h0 == kv * rep) {
-    for (uint32_t d = tid; d < D8; d += 256u) K[(uint64_t)(n - 1u) * D8 + d] = (T)(d < D ? xk[d] : 0.f);
-    for (uint32_t d = tid; d < V8; d += 256u) Vc[(uint64_t)(n - 1u) * V8 + d] = (T)(d < V ? xv[d] * iv : 0.f);
+    for (uint32_t d = tid; d < D8; d += STEP_WAVES * 64u) K[(uint64_t)(n - 1u) * D8 + d] = (T)(d < D ? xk[d] : 0.f);
+    for (uint32_t d = tid; d < V8; d += STEP_WAVES * 64u) Vc[(uint64_t)(n - 1u) * V8 + d] = (T)(d < V ? xv[d] * iv : 0.f);
   }
 }
 __global__ void __launch_bounds__(256)
@@ -202,7 +217,7 @@ k_chunk_attn_join(const ASpec s, float* act, const float* __restrict__ part, uin
     float mx = m;
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
-    const float e = lane < n_part ? expf(m - mx) : 0.f;
+    const float e = lane < n_part ? __builtin_amdgcn_exp2f(m - mx) : 0.f;
     w[lane] = e / wsumf(e * l);
   }
   __syncthreads();
@@ -361,7 +376,7 @@ k_chunk_attn_bf16(const ASpec s, float* act, const bf16_t* __restrict__ K, const
 #pragma unroll
       for (int i = 0; i < 8; i++) {
         const uint32_t d = 32u * t + 8u * kg + i;
-        const float x = d < s.dim ? xq[d] * (s.scale * 1.44269504f) : 0.f;
+        const float x = d < s.dim ? xq[d] * (s.scale * LOG2E) : 0.f;
         qh[g][t][i] = (bf16_t)x;
         ql[g][t][i] = (bf16_t)(x - (float)qh[g][t][i]);
       }
@@ -515,12 +530,12 @@ static int run_portion(const ASpec& s, float* act, T* cache, uint32_t m, uint32_
 
 template <class T, int NC, int RG, int KI>
 static int run_step_as(const ASpec& s, float* act, T* cache, uint32_t n_seq, uint32_t seq0, uint32_t pos) {
-  const uint32_t parts = cdiv(s.heads / s.kv_heads, RG), n = pos % s.chunk + 1u, unit = 16u * KI;
+  const uint32_t parts = cdiv(s.heads / s.kv_heads, RG), n = pos % s.chunk + 1u, unit = STEP_WAVES * 4u * KI;
   const uint32_t most = std::min<uint32_t>(MAX_SPANS, std::max<uint32_t>(1u, 2u * (uint32_t)g.n_cu / (s.kv_heads * parts * n_seq)));
   const uint32_t span = cdiv(cdiv(n, std::min(most, cdiv(n, unit))), unit) * unit, spans = cdiv(n, span);
   if (s.chunk > unit)      // at its full size from the first step on: a graph may be recording when the second span begins
     if (int r = scratch_need(g_parts, (size_t)n_seq * s.heads * MAX_SPANS * (s.vdim + 2) * 4)) return r;
-  k_chunk_attn_step<T, NC, RG, KI><<<dim3(s.kv_heads * parts, spans, n_seq), 256, 0, g.stream>>>(s, act, cache, (float*)g_parts.p, seq0, pos, span, parts);
+  k_chunk_attn_step<T, NC, RG, KI><<<dim3(s.kv_heads * parts, spans, n_seq), STEP_WAVES * 64, 0, g.stream>>>(s, act, cache, (float*)g_parts.p, seq0, pos, span, parts);
   count_launch();
   if (spans > 1) {
     if (int r = check_launch()) return r;
@@ -532,7 +547,7 @@ static int run_step_as(const ASpec& s, float* act, T* cache, uint32_t n_seq, uin
 template <class T>
 static int run_step(const ASpec& s, float* act, T* cache, uint32_t n_seq, uint32_t seq0, uint32_t pos) {
   const uint32_t rep = s.heads / s.kv_heads;
-  constexpr int KI = sizeof(T) == 2 ? 8 : 4;
+  constexpr int KI = 4;
   if (s.dim <= 128u && s.vdim <= 128u)
     return rep == 1 ? run_step_as<T, 1, 1, KI>(s, act, cache, n_seq, seq0, pos) : rep == 2 ? run_step_as<T, 1, 2, KI>(s, act, cache, n_seq, seq0, pos)
                                                                                           : run_step_as<T, 1, 4, KI>(s, act, cache, n_seq, seq0, pos);

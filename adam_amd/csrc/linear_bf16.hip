@@ -111,53 +111,68 @@ k_gemv_bf16(const bf16_t* __restrict__ W, float* act, const LinSpec s, uint32_t 
   __shared__ float bv[8];
   __shared__ uint32_t bi[8];
   const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, kp = s.k_stride, half = kp >> 1;
+  auto rows_of = [&](uint32_t task, uint32_t& r0, uint32_t& r1) {
+    if (EPI == LEPI_PAIR) { r0 = (task >> 4) * 32u + (task & 15u); r1 = r0 + 16u; }
+    else { r0 = task * 2u; r1 = min(r0 + 1u, s.n - 1u); }
+  };
+  uint4 p[U], q[U];
+  auto fetch = [&](uint32_t r0, uint32_t r1, uint32_t k0) {
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const uint32_t k = k0 + 512u * u;
+      p[u] = k < kp ? *(const uint4*)(W + (uint64_t)r0 * kp + k) : make_uint4(0, 0, 0, 0);
+      q[u] = k < kp ? *(const uint4*)(W + (uint64_t)r1 * kp + k) : make_uint4(0, 0, 0, 0);
+    }
+  };
+  // the first weights are on their way while x is staged, each further step's under the products of the one before
+  uint32_t task = blockIdx.x * 8u + wave, k0 = lane * 8u, r0, r1;
+  rows_of(min(task, n_tasks - 1u), r0, r1);
+  fetch(r0, r1, k0);
   operand_row<512>(s, act, row_idx ? row_idx[0] : 0u, inv, part,
                    [&](uint32_t i, float v) { xs[((i >> 2) & 1u) * half + (i >> 3) * 4u + (i & 3u)] = v; });
   __syncthreads();
-  float top = NEG_MAX_F;
+  float top = NEG_MAX_F, a0 = 0.f, a1 = 0.f;
   uint32_t top_i = 0xFFFFFFFFu;
-  for (uint32_t task = blockIdx.x * 8u + wave; task < n_tasks; task += gridDim.x * 8u) {
-    uint32_t r0, r1;
-    if (EPI == LEPI_PAIR) { r0 = (task >> 4) * 32u + (task & 15u); r1 = r0 + 16u; }
-    else { r0 = task * 2u; r1 = min(r0 + 1u, s.n - 1u); }
-    const bf16_t* w0 = W + (uint64_t)r0 * kp;
-    const bf16_t* w1 = W + (uint64_t)r1 * kp;
-    float a0 = 0.f, a1 = 0.f;
-    for (uint32_t k0 = lane * 8u; k0 < kp; k0 += 512u * U) {
-      uint4 p[U], q[U];
+  while (task < n_tasks) {
+    uint4 cp[U], cq[U];
 #pragma unroll
-      for (int u = 0; u < U; u++) {
-        const uint32_t k = k0 + 512u * u;
-        p[u] = k < kp ? *(const uint4*)(w0 + k) : make_uint4(0, 0, 0, 0);
-        q[u] = k < kp ? *(const uint4*)(w1 + k) : make_uint4(0, 0, 0, 0);
-      }
+    for (int u = 0; u < U; u++) { cp[u] = p[u]; cq[u] = q[u]; }
+    const bool last = k0 - lane * 8u + 512u * U >= kp;              // of this pair of rows
+    const uint32_t next = last ? task + gridDim.x * 8u : task, kn = last ? lane * 8u : k0 + 512u * U, c0 = r0;
+    if (next < n_tasks) {
+      if (last) rows_of(next, r0, r1);
+      fetch(r0, r1, kn);
+    }
 #pragma unroll
-      for (int u = 0; u < U; u++) {
-        const uint32_t k = k0 + 512u * u;
-        if (k >= kp) break;
-        const float4 lo = *(const float4*)(xs + (k >> 1)), hi = *(const float4*)(xs + half + (k >> 1));
-        a0 = fmaf(bf_lo(p[u].x), lo.x, a0); a1 = fmaf(bf_lo(q[u].x), lo.x, a1);
-        a0 = fmaf(bf_hi(p[u].x), lo.y, a0); a1 = fmaf(bf_hi(q[u].x), lo.y, a1);
-        a0 = fmaf(bf_lo(p[u].y), lo.z, a0); a1 = fmaf(bf_lo(q[u].y), lo.z, a1);
-        a0 = fmaf(bf_hi(p[u].y), lo.w, a0); a1 = fmaf(bf_hi(q[u].y), lo.w, a1);
-        a0 = fmaf(bf_lo(p[u].z), hi.x, a0); a1 = fmaf(bf_lo(q[u].z), hi.x, a1);
-        a0 = fmaf(bf_hi(p[u].z), hi.y, a0); a1 = fmaf(bf_hi(q[u].z), hi.y, a1);
-        a0 = fmaf(bf_lo(p[u].w), hi.z, a0); a1 = fmaf(bf_lo(q[u].w), hi.z, a1);
-        a0 = fmaf(bf_hi(p[u].w), hi.w, a0); a1 = fmaf(bf_hi(q[u].w), hi.w, a1);
-      }
+    for (int u = 0; u < U; u++) {
+      const uint32_t k = k0 + 512u * u;
+      if (k >= kp) break;
+      const float4 lo = *(const float4*)(xs + (k >> 1)), hi = *(const float4*)(xs + half + (k >> 1));
+      a0 = fmaf(bf_lo(cp[u].x), lo.x, a0); a1 = fmaf(bf_lo(cq[u].x), lo.x, a1);
+      a0 = fmaf(bf_hi(cp[u].x), lo.y, a0); a1 = fmaf(bf_hi(cq[u].x), lo.y, a1);
+      a0 = fmaf(bf_lo(cp[u].y), lo.z, a0); a1 = fmaf(bf_lo(cq[u].y), lo.z, a1);
+      a0 = fmaf(bf_hi(cp[u].y), lo.w, a0); a1 = fmaf(bf_hi(cq[u].y), lo.w, a1);
+      a0 = fmaf(bf_lo(cp[u].z), hi.x, a0); a1 = fmaf(bf_lo(cq[u].z), hi.x, a1);
+      a0 = fmaf(bf_hi(cp[u].z), hi.y, a0); a1 = fmaf(bf_hi(cq[u].z), hi.y, a1);
+      a0 = fmaf(bf_lo(cp[u].w), hi.z, a0); a1 = fmaf(bf_lo(cq[u].w), hi.z, a1);
+      a0 = fmaf(bf_hi(cp[u].w), hi.w, a0); a1 = fmaf(bf_hi(cq[u].w), hi.w, a1);
     }
-    a0 = wsum64(a0); a1 = wsum64(a1);
-    if (EPI == LEPI_PAIR) {
-      if (lane == 0) act[s.out + task] = silu_f(a0) * a1;
-    } else {
-      const uint32_t r = r0 + lane;
-      const float y = lane ? a1 : a0;
-      if (lane < 2u && r < s.n) {
-        float* d = act + s.out + r;
-        *d = EPI == LEPI_ADD ? *d + y : y;
-        if (EPI == LEPI_ARGMAX && !isnan(y) && y > top) { top = y; top_i = r; }
+    if (last) {
+      a0 = wsum64(a0); a1 = wsum64(a1);
+      if (EPI == LEPI_PAIR) {
+        if (lane == 0) act[s.out + task] = silu_f(a0) * a1;
+      } else {
+        const uint32_t r = c0 + lane;
+        const float y = lane ? a1 : a0;
+        if (lane < 2u && r < s.n) {
+          float* d = act + s.out + r;
+          *d = EPI == LEPI_ADD ? *d + y : y;
+          if (EPI == LEPI_ARGMAX && !isnan(y) && y > top) { top = y; top_i = r; }
+        }
       }
+      a0 = a1 = 0.f;
     }
+    task = next; k0 = kn;
   }
   if (EPI != LEPI_ARGMAX) return;
   const float v1 = __shfl(top, 1, 64);

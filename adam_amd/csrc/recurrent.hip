@@ -37,16 +37,17 @@ __device__ __forceinline__ float wave_add(float v) {
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
   return v;
 }
-// sums over a 256-thread workgroup of up to three values at once
+// sums over a workgroup of NW waves of up to three values at once; sh: 3 NW floats
+template <int NW>
 __device__ __forceinline__ void block_add3(float& a, float& b, float& c, float* sh) {
   a = wave_add(a); b = wave_add(b); c = wave_add(c);
   const uint32_t w = threadIdx.x >> 6;
   __syncthreads();
-  if ((threadIdx.x & 63u) == 0) { sh[w] = a; sh[4 + w] = b; sh[8 + w] = c; }
+  if ((threadIdx.x & 63u) == 0) { sh[w] = a; sh[NW + w] = b; sh[2 * NW + w] = c; }
   __syncthreads();
-  a = (sh[0] + sh[1]) + (sh[2] + sh[3]);
-  b = (sh[4] + sh[5]) + (sh[6] + sh[7]);
-  c = (sh[8] + sh[9]) + (sh[10] + sh[11]);
+  a = b = c = 0.f;
+#pragma unroll
+  for (int i = 0; i < NW; i++) { a += sh[i]; b += sh[NW + i]; c += sh[2 * NW + i]; }
 }
 
 // silu of the causal convolution at token position p for channel ch, older inputs from the ring only.  The taps' loads do
@@ -89,17 +90,15 @@ __device__ __forceinline__ void conv_silu_rows(const float* x, uint32_t x_stride
   }
 }
 
-// dot product of a bf16 matrix row with a float32 vector, by 8 neighbouring lanes (all get the sum)
-__device__ __forceinline__ float dot8(const bf16_t* w, const float* x, uint32_t k, uint32_t kp, uint32_t sub) {
+// dot product of a bf16 matrix row of kp columns (a multiple of 64, zeros at the end) with a float32 vector of as many,
+// by 8 neighbouring lanes (all get the sum)
+__device__ __forceinline__ float dot8(const bf16_t* w, const float* x, uint32_t kp, uint32_t sub) {
   float a = 0.f;
   for (uint32_t c = sub * 8u; c < kp; c += 64u) {
     const uint4 p = *(const uint4*)(w + c);
     const uint32_t u[4] = {p.x, p.y, p.z, p.w};
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-      if (c + 2 * i < k) a = fmaf(bf_lo(u[i]), x[c + 2 * i], a);
-      if (c + 2 * i + 1 < k) a = fmaf(bf_hi(u[i]), x[c + 2 * i + 1], a);
-    }
+    for (int i = 0; i < 4; i++) { a = fmaf(bf_lo(u[i]), x[c + 2 * i], a); a = fmaf(bf_hi(u[i]), x[c + 2 * i + 1], a); }
   }
   a += __shfl_xor(a, 1, 64); a += __shfl_xor(a, 2, 64); a += __shfl_xor(a, 4, 64);
   return a;
@@ -107,103 +106,107 @@ __device__ __forceinline__ float dot8(const bf16_t* w, const float* x, uint32_t 
 
 struct LowRank { uint32_t w, k, k_stride, src, src_stride, out, out_stride; };   // what a step needs of a linear spec
 
-// products of 8-lane rows held in registers: NC 16-byte words of the row per lane
+// the same for a row held in registers: NC 16-byte words of it per lane (zeros beyond the row), x as long
 template <int NC>
-__device__ __forceinline__ float dot8_regs(const uint4 (&w)[NC], const float* x, uint32_t k, uint32_t sub) {
+__device__ __forceinline__ float dot8_regs(const uint4 (&w)[NC], const float* x, uint32_t kp, uint32_t sub) {
   float a = 0.f;
 #pragma unroll
   for (int n = 0; n < NC; n++) {
     const uint32_t c = sub * 8u + 64u * n, u[4] = {w[n].x, w[n].y, w[n].z, w[n].w};
+    if (c >= kp) break;
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-      if (c + 2 * i < k) a = fmaf(bf_lo(u[i]), x[c + 2 * i], a);
-      if (c + 2 * i + 1 < k) a = fmaf(bf_hi(u[i]), x[c + 2 * i + 1], a);
-    }
+    for (int i = 0; i < 4; i++) { a = fmaf(bf_lo(u[i]), x[c + 2 * i], a); a = fmaf(bf_hi(u[i]), x[c + 2 * i + 1], a); }
   }
   a += __shfl_xor(a, 1, 64); a += __shfl_xor(a, 2, 64); a += __shfl_xor(a, 4, 64);
   return a;
 }
 
-// One token of one sequence per blockIdx.z; DN: state rows a thread holds (dim <= 8 DN); TM >= taps.  Everything a
+// One token of one sequence per blockIdx.z; DN: state rows a thread holds (dim <= 16 DN); TM >= taps.  Everything a
 // workgroup reads is asked for at the start: the state, the convolution's inputs, the rows of the low-rank factors (in
 // registers where their rank is at most 128).
+#define DSTEP 512u
 template <int DN, int TM>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(DSTEP)
 k_delta_step(const DSpec s, const LowRank da, const LowRank ga, float* act, const bf16_t* __restrict__ W, float* state, uint32_t seq0,
              uint32_t pos) {
-  constexpr int NP = DN / 4;                 // decay rows of 8 lanes: 32 a pass
+  constexpr int NP = DN / 4 > 0 ? DN / 4 : 1;          // decay rows of 8 lanes: 64 a pass
+  constexpr uint32_t NG = DSTEP / VC;
   extern __shared__ float lds[];
-  __shared__ float sh[12];
-  __shared__ float red[2][8][VC];
+  __shared__ float sh[3 * DSTEP / 64];
+  __shared__ float red[2][NG][VC];
   __shared__ float vs[VC];
   const uint32_t D = s.dim, V = s.vdim, tid = threadIdx.x, h = blockIdx.x, v0 = blockIdx.y * VC, row = blockIdx.z;
-  float *qs = lds, *ks = qs + D, *gs = ks + D, *lr = gs + D;
+  float *qs = lds, *ks = qs + D, *gs = ks + D, *la = gs + D, *lg = la + da.k_stride;
   const uint32_t n_ch = 2u * s.kv_heads * D + s.heads * V, rep = s.heads / s.kv_heads, kv = h / rep, sub = tid & 7u;
   const float* x = act + s.x + (uint64_t)row * s.x_stride;
   float* ring = state + (uint64_t)(seq0 + row) * s.seq_stride + s.conv_off;
   float* S = state + (uint64_t)(seq0 + row) * s.seq_stride + s.s_off + (uint64_t)h * D * V;
   const uint32_t qc = kv * D, kc = s.kv_heads * D + kv * D, vc = 2u * s.kv_heads * D + h * V;
-  const uint32_t col = tid & 31u, dg = tid >> 5, v = v0 + col;
+  const uint32_t col = tid & (VC - 1u), dg = tid / VC, v = v0 + col;
   const bool small = da.k_stride <= 128u && ga.k_stride <= 128u;
-  const uint32_t grow = h * V + min(v0 + (tid >> 3), V - 1u);
+  const uint32_t gt = DSTEP - 1u - tid, gv = v0 + (gt >> 3), grow = h * V + min(gv, V - 1u);   // gate rows: the last threads
   float st[DN];
 #pragma unroll
   for (int i = 0; i < DN; i++) {
-    const uint32_t d = dg + 8u * i;
+    const uint32_t d = dg + NG * i;
     st[i] = (pos != 0u && d < D && v < V) ? S[(uint64_t)d * V + v] : 0.f;
   }
+  for (uint32_t i = tid; i < da.k_stride; i += DSTEP) la[i] = i < da.k ? act[da.src + (uint64_t)row * da.src_stride + i] : 0.f;
+  for (uint32_t i = gt; i < ga.k_stride; i += DSTEP) lg[i] = i < ga.k ? act[ga.src + (uint64_t)row * ga.src_stride + i] : 0.f;
   uint4 wa[NP][2], wg[2];
-  if (small) {
+  float bias[NP];
 #pragma unroll
-    for (int i = 0; i < NP; i++) {
-      const bf16_t* w = W + da.w + (uint64_t)(h * D + min((tid >> 3) + 32u * i, D - 1u)) * da.k_stride;
+  for (int i = 0; i < NP; i++) {
+    const uint32_t r = h * D + min((tid >> 3) + 64u * i, D - 1u);
+    bias[i] = act[s.dt_bias + r];
+    if (small)
 #pragma unroll
-      for (int n = 0; n < 2; n++) wa[i][n] = sub * 8u + 64u * n < da.k_stride ? *(const uint4*)(w + sub * 8u + 64u * n) : make_uint4(0, 0, 0, 0);
-    }
+      for (int n = 0; n < 2; n++)
+        wa[i][n] = sub * 8u + 64u * n < da.k_stride ? *(const uint4*)(W + da.w + (uint64_t)r * da.k_stride + sub * 8u + 64u * n) : make_uint4(0, 0, 0, 0);
+  }
+  const float a_log = act[s.a_log + h], step = x[s.x_b + h];
+  if (small && gt < 8u * VC)
 #pragma unroll
     for (int n = 0; n < 2; n++)
-      wg[n] = sub * 8u + 64u * n < ga.k_stride ? *(const uint4*)(W + ga.w + (uint64_t)grow * ga.k_stride + sub * 8u + 64u * n) : make_uint4(0, 0, 0, 0);
-  }
-  for (uint32_t i = tid; i < da.k; i += 256u) lr[i] = act[da.src + (uint64_t)row * da.src_stride + i];
-  for (uint32_t i = tid; i < ga.k; i += 256u) lr[da.k + i] = act[ga.src + (uint64_t)row * ga.src_stride + i];
+      wg[n] = (gt & 7u) * 8u + 64u * n < ga.k_stride ? *(const uint4*)(W + ga.w + (uint64_t)grow * ga.k_stride + (gt & 7u) * 8u + 64u * n) : make_uint4(0, 0, 0, 0);
   float sq = 0.f, sk = 0.f, qk = 0.f;
-  for (uint32_t i = tid; i < 2u * D; i += 256u) {
+  for (uint32_t i = tid; i < 2u * D; i += DSTEP) {
     const bool is_k = i >= D;
     const uint32_t d = is_k ? i - D : i;
     const float a = conv_silu_ring<TM>(x, ring, n_ch, (is_k ? kc : qc) + d, pos, act + (is_k ? s.ck : s.cq) + (uint64_t)(kv * D + d) * s.taps, s.taps);
     (is_k ? ks : qs)[d] = a;
     if (is_k) sk = fmaf(a, a, sk); else sq = fmaf(a, a, sq);
   }
-  if (tid < VC && v0 + tid < V)
-    vs[tid] = conv_silu_ring<TM>(x, ring, n_ch, vc + v0 + tid, pos, act + s.cv + (uint64_t)(h * V + v0 + tid) * s.taps, s.taps);
-  const float ea = expf(act[s.a_log + h]), beta = sigmoid_f(x[s.x_b + h]);
+  if (gt < VC && v0 + gt < V)
+    vs[gt] = conv_silu_ring<TM>(x, ring, n_ch, vc + v0 + gt, pos, act + s.cv + (uint64_t)(h * V + v0 + gt) * s.taps, s.taps);
+  const float ea = expf(a_log), beta = sigmoid_f(step);
   __syncthreads();
-  for (uint32_t d = tid; d < D; d += 256u) qk = fmaf(qs[d], ks[d], qk);
+  for (uint32_t d = tid; d < D; d += DSTEP) qk = fmaf(qs[d], ks[d], qk);
   if (small) {
 #pragma unroll
     for (int i = 0; i < NP; i++) {
-      const uint32_t d = (tid >> 3) + 32u * i;
-      const float a = dot8_regs<2>(wa[i], lr, da.k, sub);
-      if (sub == 0 && d < D) gs[d] = expf(-ea * softplus_f(a + act[s.dt_bias + h * D + d]));
+      const uint32_t d = (tid >> 3) + 64u * i;
+      const float a = dot8_regs<2>(wa[i], la, da.k_stride, sub);
+      if (sub == 0 && d < D) gs[d] = expf(-ea * softplus_f(a + bias[i]));
     }
-    const float a = dot8_regs<2>(wg, lr + da.k, ga.k, sub);
-    if (sub == 0 && v0 + (tid >> 3) < V) act[ga.out + (uint64_t)row * ga.out_stride + grow] = a;
   } else {
-    for (uint32_t d = tid >> 3; d < ((D + 31u) & ~31u); d += 32u) {      // whole waves take part in the dot products
+    for (uint32_t d = tid >> 3; d < ((D + 63u) & ~63u); d += 64u) {      // whole waves take part in the dot products
       const uint32_t r = h * D + min(d, D - 1u);
-      const float a = dot8(W + da.w + (uint64_t)r * da.k_stride, lr, da.k, da.k_stride, sub);
+      const float a = dot8(W + da.w + (uint64_t)r * da.k_stride, la, da.k_stride, sub);
       if (sub == 0 && d < D) gs[d] = expf(-ea * softplus_f(a + act[s.dt_bias + r]));
     }
-    const float a = dot8(W + ga.w + (uint64_t)grow * ga.k_stride, lr + da.k, ga.k, ga.k_stride, sub);
-    if (sub == 0 && v0 + (tid >> 3) < V) act[ga.out + (uint64_t)row * ga.out_stride + grow] = a;
   }
-  block_add3(sq, sk, qk, sh);                  // (its barriers also publish gs)
+  if (gt < 8u * VC) {
+    const float a = small ? dot8_regs<2>(wg, lg, ga.k_stride, gt & 7u) : dot8(W + ga.w + (uint64_t)grow * ga.k_stride, lg, ga.k_stride, gt & 7u);
+    if ((gt & 7u) == 0 && gv < V) act[ga.out + (uint64_t)row * ga.out_stride + grow] = a;
+  }
+  block_add3<DSTEP / 64>(sq, sk, qk, sh);      // (its barriers also publish gs)
   const float iq = 1.0f / sqrtf(sq + 1e-6f) / sqrtf((float)D), ik = 1.0f / sqrtf(sk + 1e-6f);
   qk = qk * iq * ik;
   float pk = 0.f, pq = 0.f;
 #pragma unroll
   for (int i = 0; i < DN; i++) {
-    const uint32_t d = dg + 8u * i;
+    const uint32_t d = dg + NG * i;
     if (d < D) {
       st[i] *= gs[d];
       pk = fmaf(st[i], ks[d], pk); pq = fmaf(st[i], qs[d], pq);
@@ -213,20 +216,20 @@ k_delta_step(const DSpec s, const LowRank da, const LowRank ga, float* act, cons
   __syncthreads();
   pk = 0.f; pq = 0.f;
 #pragma unroll
-  for (int i = 0; i < 8; i++) { pk += red[0][i][col]; pq += red[1][i][col]; }
+  for (int i = 0; i < (int)NG; i++) { pk += red[0][i][col]; pq += red[1][i][col]; }
   if (v < V) {
     const float u = beta * (vs[col] - pk * ik);
     if (dg == 0) act[s.out + (uint64_t)row * s.out_stride + h * V + v] = fmaf(u, qk, pq * iq);
     const float uk = u * ik;
 #pragma unroll
     for (int i = 0; i < DN; i++) {
-      const uint32_t d = dg + 8u * i;
+      const uint32_t d = dg + NG * i;
       if (d < D) S[(uint64_t)d * V + v] = fmaf(ks[d], uk, st[i]);
     }
   }
   float* slot = ring + (uint64_t)(pos % s.taps) * n_ch;
   if (blockIdx.y == 0 && h % rep == 0)
-    for (uint32_t d = tid; d < D; d += 256u) { slot[qc + d] = x[qc + d]; slot[kc + d] = x[kc + d]; }
+    for (uint32_t d = tid; d < D; d += DSTEP) { slot[qc + d] = x[qc + d]; slot[kc + d] = x[kc + d]; }
   if (tid < VC && v0 + tid < V) slot[vc + v0 + tid] = x[vc + v0 + tid];
 }
 
@@ -264,7 +267,7 @@ k_retention_step(const RSpec s, float* act, float* state, uint32_t seq0, uint32_
     ks[d] = rotated(x + s.x_k + h * D, act + s.freq, d, s.rot_dims, pos) * kscale;
     qk = fmaf(qs[d], ks[d], qk);
   }
-  block_add3(qk, z0, z1, sh);
+  block_add3<4>(qk, z0, z1, sh);
   float pq = 0.f;
 #pragma unroll
   for (int i = 0; i < DN; i++) {
@@ -636,13 +639,13 @@ int adamah_delta_rule_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, 
   }
   float *act = (float*)ma->buf, *state = (float*)ms->buf;
   if (rows == 1) {
-    const size_t lds = (size_t)(3 * D + da->k + ga->k) * 4;
+    const size_t lds = (size_t)(3 * D + da->k_stride + ga->k_stride) * 4;
     if (lds > 48000) return ADAMAH_ERR_INVALID;
     const dim3 grid((uint32_t)H, cdiv(V, VC), n_seq);
     const bf16_t* W = (const bf16_t*)mw->buf;
-#define STEP(DN, TM) k_delta_step<DN, TM><<<grid, 256, lds, g.stream>>>(*s, low_rank(*da), low_rank(*ga), act, W, state, seq0, pos)
-    if (s->taps <= 4) { if (D <= 64) STEP(8, 4); else if (D <= 128) STEP(16, 4); else STEP(32, 4); }
-    else { if (D <= 64) STEP(8, MAX_TAPS); else if (D <= 128) STEP(16, MAX_TAPS); else STEP(32, MAX_TAPS); }
+#define STEP(DN, TM) k_delta_step<DN, TM><<<grid, DSTEP, lds, g.stream>>>(*s, low_rank(*da), low_rank(*ga), act, W, state, seq0, pos)
+    if (s->taps <= 4) { if (D <= 64) STEP(4, 4); else if (D <= 128) STEP(8, 4); else STEP(16, 4); }
+    else { if (D <= 64) STEP(4, MAX_TAPS); else if (D <= 128) STEP(8, MAX_TAPS); else STEP(16, MAX_TAPS); }
 #undef STEP
     count_launch();
     return check_launch();
