@@ -270,14 +270,24 @@ k_linear_skinny(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X, floa
   f4_t acc[2][MT];
 #pragma unroll
   for (int m = 0; m < MT; m++) { acc[0][m] = (f4_t){0, 0, 0, 0}; acc[1][m] = (f4_t){0, 0, 0, 0}; }
-#pragma unroll 4
-  for (uint32_t k = wave * 32u; k < kp; k += 256u) {
-    const bf8_t a = *(const bf8_t*)(wa + k), b = *(const bf8_t*)(wb + k);
+  constexpr int UN = 4;                                // K steps in flight
+  for (uint32_t k0 = wave * 32u; k0 < kp; k0 += 256u * UN) {
+    bf8_t a[UN], b[UN], x[UN][MT];
 #pragma unroll
-    for (int m = 0; m < MT; m++) {
-      const bf8_t x = *(const bf8_t*)(xr[m] + k);
-      acc[0][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, x, acc[0][m], 0, 0, 0);
-      acc[1][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b, x, acc[1][m], 0, 0, 0);
+    for (int u = 0; u < UN; u++) {
+      const uint32_t k = min(k0 + 256u * u, kp - 32u);
+      a[u] = *(const bf8_t*)(wa + k); b[u] = *(const bf8_t*)(wb + k);
+#pragma unroll
+      for (int m = 0; m < MT; m++) x[u][m] = *(const bf8_t*)(xr[m] + k);
+    }
+#pragma unroll
+    for (int u = 0; u < UN; u++) {
+      if (k0 + 256u * u >= kp) break;
+#pragma unroll
+      for (int m = 0; m < MT; m++) {
+        acc[0][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u], x[u][m], acc[0][m], 0, 0, 0);
+        acc[1][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b[u], x[u][m], acc[1][m], 0, 0, 0);
+      }
     }
   }
 #pragma unroll

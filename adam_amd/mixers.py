@@ -20,6 +20,21 @@ from dataclasses import dataclass
 import numpy as np
 
 
+MAX_DIM, MAX_TAPS = 256, 16            # what the kernels hold of a head in registers and shared memory
+
+
+def _fits(name, **dims):
+    for n, v in dims.items():
+        top = MAX_TAPS if n == "conv" else MAX_DIM
+        if not 1 <= v <= top:
+            raise ValueError(f"{name}: {n} = {v} is outside 1 .. {top}")
+
+
+def _grouped(name, heads, kv_heads):
+    if kv_heads < 1 or heads % kv_heads:
+        raise ValueError(f"{name}: {heads} heads do not share {kv_heads} key heads evenly")
+
+
 @dataclass
 class ChannelDelta:
     """Gated delta rule: short convolutions on q, k, v, unit q and k, one decay per head and key channel (low-rank),
@@ -33,6 +48,10 @@ class ChannelDelta:
     @classmethod
     def from_config(cls, d):
         return cls(*(int(d[n]) for n in ("heads", "kv_heads", "dim", "vdim", "conv")))
+
+    def __post_init__(self):
+        _fits("delta rule", dim=self.dim, vdim=self.vdim, conv=self.conv)
+        _grouped("delta rule", self.heads, self.kv_heads)
 
     def tensors(self, E):
         H, KH, D, V, T = self.heads, self.kv_heads, self.dim, self.vdim, self.conv
@@ -98,6 +117,12 @@ class ChunkAttention:
         return cls(int(d["heads"]), int(d["kv_heads"]), int(d["dim"]), int(d["vdim"]), float(d["scale"]),
                    int(d["mask"]["size"]), rows)
 
+    def __post_init__(self):
+        _fits("chunk attention", dim=self.dim, vdim=self.vdim)
+        _grouped("chunk attention", self.heads, self.kv_heads)
+        if self.chunk < 1:
+            raise ValueError(f"chunk attention: a chunk of {self.chunk} tokens")
+
     def tensors(self, E):
         H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
         return {"q": (H * D, E), "k": (G * D, E), "v": (G * V, E), "o": (E, H * V), "r1": (H,), "r2": (H,)}
@@ -149,11 +174,15 @@ class Retention:
 
     @classmethod
     def from_config(cls, d, rows="o"):
-        c = cls(int(d["heads"]), int(d["dim"]), int(d["vdim"]), tuple(float(v) for v in d["decay"]), float(d["rot"]["base"]),
-                int(d["rot"]["dims"]), rows)
-        if len(c.decay) != c.heads:
-            raise ValueError(f"retention: {len(c.decay)} decays for {c.heads} heads")
-        return c
+        return cls(int(d["heads"]), int(d["dim"]), int(d["vdim"]), tuple(float(v) for v in d["decay"]), float(d["rot"]["base"]),
+                   int(d["rot"]["dims"]), rows)
+
+    def __post_init__(self):
+        _fits("retention", dim=self.dim, vdim=self.vdim)
+        if len(self.decay) != self.heads:
+            raise ValueError(f"retention: {len(self.decay)} decays for {self.heads} heads")
+        if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
+            raise ValueError(f"retention: {self.rot_dims} rotated dimensions of {self.dim}")
 
     def tensors(self, E):
         H, D, V = self.heads, self.dim, self.vdim

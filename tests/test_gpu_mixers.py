@@ -65,7 +65,8 @@ class Pair:
 @pytest.mark.parametrize("rows,n,k,groups,epi", [
     (1, 70, 33, 3, 0), (1, 96, 640, 0, 2), (1, 51, 1100, 1, 1), (1, 33, 1536, 32, 0), (2, 70, 33, 3, 0), (5, 64, 200, 5, 2),
     (16, 129, 64, 1, 1), (17, 64, 320, 2, 2), (31, 45, 96, 0, 0), (33, 96, 130, 13, 2), (64, 200, 256, 4, 1), (65, 130, 72, 0, 0),
-    (200, 1000, 192, 3, 0), (300, 8224, 64, 1, 2), (300, 8200, 128, 1, 1)])
+    (200, 1000, 192, 3, 0), (300, 8224, 64, 1, 2), (300, 8200, 128, 1, 1),
+    (1, 10, 20000, 4, 0), (3, 37, 16000, 4, 0)])
 def test_linear(hip, dtype, rows, n, k, groups, epi):
     note(f"linear {dtype} rows {rows} n {n} k {k} groups {groups} epi {epi}")
     rng = np.random.default_rng(rows * 1000 + n)
@@ -168,7 +169,8 @@ def delta_pair(hip, H, KH, D, V, taps, rank, rows, seqs, strong, seed):
 
 @pytest.mark.parametrize("H,KH,D,V,taps,rank,strong", [
     (4, 2, 24, 20, 4, 11, False), (3, 3, 17, 33, 3, 5, True), (1, 1, 1, 1, 1, 1, False), (2, 1, 64, 16, 2, 70, True),
-    (2, 2, 128, 144, 5, 16, False), (2, 1, 200, 40, 4, 128, True), (2, 1, 256, 64, 8, 30, False)])
+    (2, 2, 128, 144, 5, 16, False), (2, 1, 200, 40, 4, 128, True), (2, 1, 256, 64, 8, 30, False),
+    (1, 1, 256, 250, 16, 20, False)])
 def test_delta_rule(hip, H, KH, D, V, taps, rank, strong):
     note(f"delta rule H {H} KH {KH} D {D} V {V} taps {taps} rank {rank}")
     run = delta_pair(hip, H, KH, D, V, taps, rank, 40, 3, strong, seed=D)

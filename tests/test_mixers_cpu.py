@@ -162,6 +162,29 @@ def test_wrong_files_fail_by_name(tmp_path):
             load_config(str(tmp_path))
 
 
+def test_sizes_the_kernels_do_not_hold_are_refused_at_load():
+    bad = [delta(dim=300), delta(conv=17), delta(heads=4, kv_heads=3), par(size=0), par(rot=13), par(r_heads=2, decay=[0.5]), par(r_vdim=257)]
+    for layer in bad:
+        with pytest.raises(ValueError):
+            vomotar_config(config([layer]))
+    with pytest.raises(ValueError, match="groups"):
+        vomotar_config(config([delta()], width=50, groups=4))
+
+
+def test_specs_agree_with_the_header_and_the_numpy_surface():
+    """The structs that travel in handles: same fields in the same order, in C, in the binding and in the oracle."""
+    import re
+    from oracle import mixer_ops_np as O
+    src = re.sub(r"/\*.*?\*/", "", open(os.path.join(os.path.dirname(A.__file__), "..", "include", "adamah_hip.h")).read(), flags=re.S)
+    for c_name, cls, fields in (("AdamahLinearSpec", A.LinearSpec, O._LINEAR), ("AdamahMergeSpec", A.MergeSpec, O._MERGE),
+                                ("AdamahDeltaSpec", A.DeltaSpec, O._DELTA), ("AdamahRetentionSpec", A.RetentionSpec, O._RET),
+                                ("AdamahChunkAttnSpec", A.ChunkAttnSpec, O._ATT)):
+        body = re.search(r"typedef struct %s \{(.*?)\}" % c_name, src, flags=re.S).group(1)
+        decl = [(t, n.strip()) for t, names in re.findall(r"(uint32_t|float)([^;]*);", body) for n in names.split(",")]
+        ours = [("float" if t is A.f32c else "uint32_t", n) for n, t in cls._fields_]
+        assert decl == ours and [n for _, n in ours] == fields.split(), c_name
+
+
 def test_bfloat16_rounding():
     x = np.array([1.0, 1.00390625, 1.01171875, -3.1415927, 65504.0, 1e-30, np.inf], np.float32)
     r = bf16_to_f32(f32_to_bf16(x))
