@@ -223,7 +223,7 @@ class Retention:
 
 @dataclass
 class Parallel:
-    """Two mixers that read the same row; half the sum of their outputs, each normed over the model width."""
+    """Mean of two branches over the same input, each through a full-width RMS norm with a weight of its own."""
     left: object
     right: object
 

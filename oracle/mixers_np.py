@@ -126,7 +126,7 @@ def sub(W, prefix):
 
 
 def parallel(h, W, c, eps, plant=None):
-    """Half the sum of the two mixers' outputs, each normed over the model width with its own weight."""
+    """Mean of two branches over the same input; a branch passes through a full-width RMS norm first."""
     left = chunk_attention(h, sub(W, 'left.'), c['left'], eps, plant)
     right = retention(h, sub(W, 'right.'), c['right'], eps)
     return 0.5 * (rms(left, eps) * W['left.out'] + rms(right, eps) * W['right.out'])
