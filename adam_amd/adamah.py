@@ -38,7 +38,7 @@ DECODE_RUNTIME_SEQ_LEN = 0xFFFFFFFD
  DECODE_OP_FUSED_GATEUP_ACT_T_XQ8) = range(26, 31)
 # layered mixers over bfloat16 weights (no counterpart in the reference)
 (DECODE_OP_LINEAR, DECODE_OP_LINEAR_ARGMAX, DECODE_OP_MERGE_NORM, DECODE_OP_DELTA_RULE, DECODE_OP_RETENTION,
- DECODE_OP_CHUNK_ATTENTION) = range(31, 37)
+ DECODE_OP_CHUNK_ATTENTION, DECODE_OP_WINDOW_ATTENTION, DECODE_OP_STATE_SPACE, DECODE_OP_EXPERTS) = range(31, 40)
 
 (OP_NEG, OP_ABS, OP_SQRT, OP_EXP, OP_LOG, OP_TANH, OP_RELU, OP_GELU, OP_SIN, OP_COS, OP_TAN, OP_ASIN,
  OP_ACOS, OP_ATAN, OP_SINH, OP_COSH, OP_SIGMOID, OP_SWISH, OP_MISH, OP_SELU, OP_ELU, OP_LEAKY_RELU,
@@ -67,15 +67,25 @@ def _spec(name, fields, floats=()):
 
 
 LinearSpec = _spec("LinearSpec", "w n k k_stride src src_stride groups eps wt wt_len gate gate_stride gate_act opnd ready out "
-                   "out_stride epi out_opnd out_opnd_stride", ("eps",))
-MergeSpec = _spec("MergeSpec", "a b stride wa wb dst dst_stride dim eps scale", ("eps", "scale"))
+                   "out_stride epi out_opnd out_opnd_stride wt_add bias biased branch branch_stride branch_wt branched res_out res_stride "
+                   "keep keep_stride kept tail tail_out tail_stride", ("eps", "wt_add"))
+MergeSpec = _spec("MergeSpec", "a b stride wa wb dst dst_stride dim eps scale store", ("eps", "scale"))
 DeltaSpec = _spec("DeltaSpec", "heads kv_heads dim vdim taps x x_stride x_b cq ck cv a_log dt_bias out out_stride state_map s_off "
                   "conv_off seq_stride")
 RetentionSpec = _spec("RetentionSpec", "heads dim vdim rot_dims freq decay x x_stride x_q x_k x_v out out_stride state_map s_off "
                       "seq_stride")
 ChunkAttnSpec = _spec("ChunkAttnSpec", "heads kv_heads dim vdim chunk x x_stride x_q x_k x_v r1 r2 scale eps out out_stride "
                       "cache_map k_off v_off seq_stride", ("scale", "eps"))
-GATE_NONE, GATE_SIGMOID, GATE_SILU = 0, 1, 2
+WindowAttnSpec = _spec("WindowAttnSpec", "heads kv_heads dim vdim window x x_stride x_q x_k x_v slope sink has_sink qk_norm scale eps "
+                       "softcap temp_coef temp_every out out_stride cache_map k_off v_off seq_stride",
+                       ("scale", "eps", "softcap", "temp_coef"))
+StateSpaceSpec = _spec("StateSpaceSpec", "heads groups state vdim taps x x_stride x_c x_dt conv conv_b dt_bias a_log skip out out_stride "
+                       "state_map s_off conv_off seq_stride")
+ExpertsSpec = _spec("ExpertsSpec", "experts identity top ff ff_stride width k_stride gate_up gate_up_step down down_step logits "
+                    "logits_stride correction x x_stride opnd act act_opnd shared_ff shared_ff_stride shared_down shared_act out "
+                    "out_stride epi")
+BigramSpec = _spec("BigramSpec", "table vocab width dst scale pairs buckets mul_prev mul_cur state_map prev_off seq_stride", ("scale",))
+GATE_NONE, GATE_SIGMOID, GATE_SILU, GATE_SILU_AHEAD = 0, 1, 2, 3
 EPI_STORE, EPI_ADD, EPI_SWIGLU = 0, 1, 2
 
 
@@ -159,7 +169,9 @@ _SIGS = {
     "map_fused_gateup_act_t_xq8_dev": (i32, [_U] * 8),
     "adamah_linear_dev": (i32, [_U] * 6), "adamah_linear_argmax_dev": (i32, [_U] * 6), "adamah_merge_norm_dev": (i32, [_U] * 3),
     "adamah_delta_rule_dev": (i32, [_U] * 10), "adamah_retention_dev": (i32, [_U] * 6),
-    "adamah_chunk_attention_dev": (i32, [_U] * 6),
+    "adamah_chunk_attention_dev": (i32, [_U] * 6), "adamah_window_attention_dev": (i32, [_U] * 6),
+    "adamah_state_space_dev": (i32, [_U] * 6), "adamah_experts_dev": (i32, [_U] * 6),
+    "adamah_hip_embed_bigram_dev": (i32, [_U] * 8 + [pu32]),
     # timing helpers for benchmarks (HIP events on the library's own stream)
     "adamah_hip_timer_begin": (i32, []), "adamah_hip_timer_end": (f32c, []),
     "adamah_hip_debug_dequant": (i32, [_U, u64, u64, pf32]),
@@ -752,6 +764,23 @@ class Adamah:
 
     def chunk_attention_dev(self, map_act, spec_handle, n_seq, rows, seq0, pos):
         self._op("adamah_chunk_attention_dev", map_act, spec_handle, n_seq, rows, seq0, pos)
+
+    def window_attention_dev(self, map_act, spec_handle, n_seq, rows, seq0, pos):
+        self._op("adamah_window_attention_dev", map_act, spec_handle, n_seq, rows, seq0, pos)
+
+    def state_space_dev(self, map_act, spec_handle, n_seq, rows, seq0, pos):
+        self._op("adamah_state_space_dev", map_act, spec_handle, n_seq, rows, seq0, pos)
+
+    def experts_dev(self, map_act, map_opnd, map_wt, spec_handle, shared_handle, rows):
+        self._op("adamah_experts_dev", map_act, map_opnd, map_wt, spec_handle, shared_handle, rows)
+
+    def embed_bigram_dev(self, map_act, map_src, spec_handle, locs_tokens_handle, n_seq, rows, seq0, pos, post=False):
+        """Embedding rows with the bigram table; `post`: the launch also hands the token values to the host and the ticket
+        to wait on comes back."""
+        t = ctypes.c_uint32(0)
+        self._op("adamah_hip_embed_bigram_dev", map_act, map_src, spec_handle, locs_tokens_handle, n_seq, rows, seq0, pos,
+                 ctypes.byref(t) if post else None)
+        return t.value
 
     # ---- benchmark / test helpers (not part of the reference surface) ------------------
     def timer_begin(self):

@@ -201,9 +201,11 @@ int launch_attn_combine_dev(Map* m, const float* partial, const uint32_t* lo_dev
                             uint32_t n_splits);
 void attn_decode_release();
 void attn_prefill_release();   // attn_prefill.hip: the transposed V tiles (shutdown)
-void linear_release();          // linear_bf16.hip, recurrent.hip, attn_chunk.hip: their scratch (shutdown)
+void linear_release();          // linear_bf16.hip, recurrent.hip, state_space.hip, attn_bounded.hip, experts.hip: their scratch (shutdown)
 void recurrent_release();
-void attn_chunk_release();
+void state_space_release();
+void experts_release();
+void attn_bounded_release();
 void token_feed_release();      // frees the pinned ring tokens reach the host through (shutdown)
 
 inline void layout_changed() { g.layout_gen++; }

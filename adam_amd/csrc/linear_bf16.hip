@@ -1,4 +1,5 @@
-// y = W . f(x) over bfloat16 weight maps, f a grouped RMSNorm (with weight and gate) or nothing.
+// y = W . f(x) over bfloat16 weight maps, f a grouped RMSNorm (with weight and gate; of one row or of the sum of a row and
+// a normed one) or nothing.
 //
 //   one row      k_gemv_bf16: f is computed by every workgroup while it stages x in LDS (float32), weights stream
 //                through registers, float32 multiply-adds; store, add to the residual, gate / up pairs combined, or
@@ -33,67 +34,125 @@ void scratch_free(Scratch& s) {
   s.p = nullptr; s.cap = 0;
 }
 
-__device__ __forceinline__ float wsum64(float v) {
+// Sum over a workgroup of NW waves; sh: NW floats that no earlier sum still reads.
+template <int NW>
+__device__ __forceinline__ float block_sum(float v, float* sh) {
+  v = wsum64(v);
+  if ((threadIdx.x & 63u) == 0) sh[threadIdx.x >> 6] = v;
+  __syncthreads();
+  v = 0.f;
 #pragma unroll
-  for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+  for (int w = 0; w < NW; w++) v += sh[w];
   return v;
 }
-
-// f(x) of one row by a workgroup of NT threads; put(i, value) for i in [0, k_stride).  inv: LDS, LIN_MAX_GROUPS floats,
-// part: LDS, 2 NT / 64 floats.
-template <int NT, class Put>
-__device__ __forceinline__ void operand_row(const LinSpec& s, const float* __restrict__ act, uint32_t row, float* inv,
-                                            float* part, Put put) {
+// Root mean squares of the row's groups -> inv (with a barrier behind them).
+template <int NT, class Val>
+__device__ __forceinline__ void group_inverse(const LinSpec& s, float* inv, float* part, Val val) {
   constexpr uint32_t NW = NT / 64;
-  const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6;
-  const float* x = act + s.src + (uint64_t)row * s.src_stride;
-  if (s.groups) {
-    const uint32_t gs = s.k / s.groups;
-    if (s.groups >= NW) {
-      for (uint32_t gi = wave; gi < s.groups; gi += NW) {
-        float ss = 0.f;
-        for (uint32_t i = lane; i < gs; i += 64u) { const float v = x[gi * gs + i]; ss = fmaf(v, v, ss); }
-        ss = wsum64(ss);
-        if (lane == 0) inv[gi] = 1.0f / sqrtf(ss / (float)gs + s.eps);
-      }
-      __syncthreads();
-    } else {                                    // fewer groups than waves: `sub` waves share a group
-      const uint32_t sub = NW / s.groups, gi = wave / sub, sp = wave % sub;
+  const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, gs = s.k / s.groups;
+  if (s.groups >= NW) {
+    for (uint32_t gi = wave; gi < s.groups; gi += NW) {
       float ss = 0.f;
-      if (gi < s.groups)
-        for (uint32_t i = sp * 64u + lane; i < gs; i += sub * 64u) { const float v = x[gi * gs + i]; ss = fmaf(v, v, ss); }
+      for (uint32_t i = lane; i < gs; i += 64u) { const float v = val(gi * gs + i); ss = fmaf(v, v, ss); }
       ss = wsum64(ss);
-      if (lane == 0) part[wave] = ss;
-      __syncthreads();
-      if (tid < s.groups) {
-        float t = 0.f;
-        for (uint32_t j = 0; j < sub; j++) t += part[tid * sub + j];
-        inv[tid] = 1.0f / sqrtf(t / (float)gs + s.eps);
-      }
-      __syncthreads();
+      if (lane == 0) inv[gi] = 1.0f / sqrtf(ss / (float)gs + s.eps);
     }
-    const float* wt = act + s.wt;
+    __syncthreads();
+  } else {                                    // fewer groups than waves: `sub` waves share a group
+    const uint32_t sub = NW / s.groups, gi = wave / sub, sp = wave % sub;
+    float ss = 0.f;
+    if (gi < s.groups)
+      for (uint32_t i = sp * 64u + lane; i < gs; i += sub * 64u) { const float v = val(gi * gs + i); ss = fmaf(v, v, ss); }
+    ss = wsum64(ss);
+    if (lane == 0) part[wave] = ss;
+    __syncthreads();
+    if (tid < s.groups) {
+      float t = 0.f;
+      for (uint32_t j = 0; j < sub; j++) t += part[tid * sub + j];
+      inv[tid] = 1.0f / sqrtf(t / (float)gs + s.eps);
+    }
+    __syncthreads();
+  }
+}
+// f(x) of one row by a workgroup of NT threads; put(i, value) for i in [0, k_stride).  first: this workgroup also stores
+// what the spec wants kept.  inv: LDS, LIN_MAX_GROUPS floats, part: LDS, 2 NT / 64 floats.
+template <int NT, class Put>
+__device__ __forceinline__ void operand_row(const LinSpec& s, float* act, uint32_t row, bool first, float* inv, float* part, Put put) {
+  const uint32_t tid = threadIdx.x;
+  const float* x = act + s.src + (uint64_t)row * s.src_stride;
+  float* keep = act + s.keep + (uint64_t)row * s.keep_stride;
+  const bool kept = first && s.kept;
+  const float* wt = act + s.wt;
+  if (s.branched) {
+    // x + the branch's row behind a norm of its own: eight elements a thread stay in registers (a longer row is read again)
+    constexpr int R = 8;
+    const float *b = act + s.branch + (uint64_t)row * s.branch_stride, *bw = act + s.branch_wt;
+    float* res = act + s.res_out + (uint64_t)row * s.res_stride;
+    float xv[R], bv[R], wv[R], nv[R], ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+      const uint32_t i = tid + (uint32_t)j * NT;
+      const bool on = i < s.k;
+      bv[j] = on ? b[i] : 0.f; xv[j] = on ? x[i] : 0.f; wv[j] = on ? bw[i] : 0.f; nv[j] = on && s.wt_len ? wt[i] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < R; j++) ss = fmaf(bv[j], bv[j], ss);
+    for (uint32_t i = tid + (uint32_t)R * NT; i < s.k; i += NT) ss = fmaf(b[i], b[i], ss);
+    const float ib = 1.0f / sqrtf(block_sum<NT / 64>(ss, part) / (float)s.k + s.eps);
+    ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+      const uint32_t i = tid + (uint32_t)j * NT;
+      xv[j] = fmaf(bv[j] * ib, s.wt_add + wv[j], xv[j]);
+      if (i < s.k) ss = fmaf(xv[j], xv[j], ss);
+    }
+    const auto sum_at = [&](uint32_t i) { return fmaf(b[i] * ib, s.wt_add + bw[i], x[i]); };
+    for (uint32_t i = tid + (uint32_t)R * NT; i < s.k; i += NT) { const float v = sum_at(i); ss = fmaf(v, v, ss); }
+    const float ix = 1.0f / sqrtf(block_sum<NT / 64>(ss, part + NT / 64) / (float)s.k + s.eps);
+    const auto done = [&](uint32_t i, float v, float w) {
+      if (first && s.branched == 2u) res[i] = v;
+      v *= ix;
+      if (s.wt_len) v *= s.wt_add + w;
+      if (kept) keep[i] = v;
+      put(i, v);
+    };
+#pragma unroll
+    for (int j = 0; j < R; j++) {
+      const uint32_t i = tid + (uint32_t)j * NT;
+      if (i < s.k) done(i, xv[j], nv[j]);
+    }
+    for (uint32_t i = tid + (uint32_t)R * NT; i < s.k; i += NT) done(i, sum_at(i), s.wt_len ? wt[i] : 0.f);
+  } else if (s.groups) {
+    const uint32_t gs = s.k / s.groups;
     const float* gt = act + s.gate + (uint64_t)row * s.gate_stride;
+    if (s.gate_act == 3u) group_inverse<NT>(s, inv, part, [&](uint32_t i) { return x[i] * silu_f(gt[i]); });
+    else group_inverse<NT>(s, inv, part, [&](uint32_t i) { return x[i]; });
     for (uint32_t i = tid; i < s.k; i += NT) {
-      float v = x[i] * inv[i / gs];
-      if (s.wt_len) v *= wt[s.wt_len == s.k ? i : i % s.wt_len];
+      float v = x[i];
+      if (s.gate_act == 3u) v *= silu_f(gt[i]);
+      v *= inv[i / gs];
+      if (s.wt_len) v *= s.wt_add + wt[s.wt_len == s.k ? i : i % s.wt_len];
       if (s.gate_act == 1u) v *= sigmoid_f(gt[i]);
       else if (s.gate_act == 2u) v *= silu_f(gt[i]);
+      if (kept) keep[i] = v;
       put(i, v);
     }
   } else {
-    for (uint32_t i = tid; i < s.k; i += NT) put(i, x[i]);
+    for (uint32_t i = tid; i < s.k; i += NT) {
+      if (kept) keep[i] = x[i];
+      put(i, x[i]);
+    }
   }
   for (uint32_t i = s.k + tid; i < s.k_stride; i += NT) put(i, 0.f);
 }
 
 template <class T>
 __global__ void __launch_bounds__(256)
-k_operand_rows(const LinSpec s, const float* __restrict__ act, T* __restrict__ dst, const uint32_t* __restrict__ row_idx) {
+k_operand_rows(const LinSpec s, float* act, T* __restrict__ dst, const uint32_t* __restrict__ row_idx) {
   __shared__ float inv[LIN_MAX_GROUPS];
   __shared__ float part[8];
   T* d = dst + (uint64_t)blockIdx.x * s.k_stride;
-  operand_row<256>(s, act, row_idx ? row_idx[blockIdx.x] : blockIdx.x, inv, part, [&](uint32_t i, float v) { d[i] = (T)v; });
+  operand_row<256>(s, act, row_idx ? row_idx[blockIdx.x] : blockIdx.x, true, inv, part, [&](uint32_t i, float v) { d[i] = (T)v; });
 }
 
 // ---- one row ------------------------------------------------------------------------------------------------------
@@ -111,9 +170,10 @@ k_gemv_bf16(const bf16_t* __restrict__ W, float* act, const LinSpec s, uint32_t 
   __shared__ float bv[8];
   __shared__ uint32_t bi[8];
   const uint32_t lane = threadIdx.x & 63u, wave = threadIdx.x >> 6, kp = s.k_stride, half = kp >> 1;
+  const uint32_t pairs = EPI == LEPI_PAIR ? (s.n - s.tail) >> 1 : 0u;        // the tail's rows come two a task behind the pairs
   auto rows_of = [&](uint32_t task, uint32_t& r0, uint32_t& r1) {
-    if (EPI == LEPI_PAIR) { r0 = (task >> 4) * 32u + (task & 15u); r1 = r0 + 16u; }
-    else { r0 = task * 2u; r1 = min(r0 + 1u, s.n - 1u); }
+    if (EPI == LEPI_PAIR && task < pairs) { r0 = (task >> 4) * 32u + (task & 15u); r1 = r0 + 16u; }
+    else { r0 = task * 2u; r1 = min(r0 + 1u, s.n - 1u); }     // (2 pairs + 2 (task - pairs) for the tail)
   };
   uint4 p[U], q[U];
   auto fetch = [&](uint32_t r0, uint32_t r1, uint32_t k0) {
@@ -128,7 +188,7 @@ k_gemv_bf16(const bf16_t* __restrict__ W, float* act, const LinSpec s, uint32_t 
   uint32_t task = blockIdx.x * 8u + wave, k0 = lane * 8u, r0, r1;
   rows_of(min(task, n_tasks - 1u), r0, r1);
   fetch(r0, r1, k0);
-  operand_row<512>(s, act, row_idx ? row_idx[0] : 0u, inv, part,
+  operand_row<512>(s, act, row_idx ? row_idx[0] : 0u, blockIdx.x == 0u, inv, part,
                    [&](uint32_t i, float v) { xs[((i >> 2) & 1u) * half + (i >> 3) * 4u + (i & 3u)] = v; });
   __syncthreads();
   float top = NEG_MAX_F, a0 = 0.f, a1 = 0.f;
@@ -159,13 +219,14 @@ k_gemv_bf16(const bf16_t* __restrict__ W, float* act, const LinSpec s, uint32_t 
     }
     if (last) {
       a0 = wsum64(a0); a1 = wsum64(a1);
-      if (EPI == LEPI_PAIR) {
+      if (EPI == LEPI_PAIR && task < pairs) {
         if (lane == 0) act[s.out + task] = silu_f(a0) * a1;
       } else {
         const uint32_t r = c0 + lane;
-        const float y = lane ? a1 : a0;
+        float y = lane ? a1 : a0;
         if (lane < 2u && r < s.n) {
-          float* d = act + s.out + r;
+          if (s.biased) y += act[s.bias + r];
+          float* d = EPI == LEPI_PAIR ? act + s.tail_out + (r - 2u * pairs) : act + s.out + r;
           *d = EPI == LEPI_ADD ? *d + y : y;
           if (EPI == LEPI_ARGMAX && !isnan(y) && y > top) { top = y; top_i = r; }
         }
@@ -234,9 +295,12 @@ k_best_row(const float* __restrict__ act, uint64_t src, uint32_t stride, uint32_
 
 // ---- results of the matrix-instruction kernels --------------------------------------------------------------------
 // Lane l of a 16 x 16 result holds matrix rows (outputs) 4 (l / 16) + 0..3 of token l % 16.
-template <class T>
 __device__ __forceinline__ void put_out(const LinSpec& s, float* act, uint32_t row, uint32_t n0, f4_t v) {
   float* d = act + s.out + (uint64_t)row * s.out_stride + n0;
+  if (s.biased) {
+#pragma unroll
+    for (int i = 0; i < 4; i++) if (n0 + i < s.n) v[i] += act[s.bias + n0 + i];
+  }
   if (s.epi == 1u) {
 #pragma unroll
     for (int i = 0; i < 4; i++) if (n0 + i < s.n) d[i] += v[i];
@@ -252,6 +316,18 @@ __device__ __forceinline__ void put_pair(const LinSpec& s, T* opnd, uint32_t row
   T* d = opnd + s.out_opnd + (uint64_t)row * s.out_opnd_stride + c;
 #pragma unroll
   for (int i = 0; i < 4; i++) if (n0 + i < s.n) d[i] = (T)(silu_f(gt[i]) * up[i]);
+}
+// two neighbouring runs of 16 rows of an epi 2 product, from row n0 on: a pair, or two runs of the tail
+template <class T>
+__device__ __forceinline__ void put_pair_or_tail(const LinSpec& s, float* act, T* opnd, uint32_t row, uint32_t n0, f4_t a, f4_t b) {
+  const uint32_t head = s.n - s.tail;
+  if (n0 < head) { put_pair(s, opnd, row, n0, a, b); return; }
+  float* d = act + s.tail_out + (uint64_t)row * s.tail_stride + (n0 - head);
+#pragma unroll
+  for (int i = 0; i < 4; i++) {
+    if (n0 + i < s.n) d[i] = a[i];
+    if (n0 + 16u + i < s.n) d[16 + i] = b[i];
+  }
 }
 
 // ---- 2 .. 32 rows -------------------------------------------------------------------------------------------------
@@ -298,36 +374,22 @@ k_linear_skinny(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X, floa
       f4_t gt = red[0][wave][lane], up = red[0][MT + wave][lane];
       for (int w = 1; w < 8; w++) { gt += red[w][wave][lane]; up += red[w][MT + wave][lane]; }
       const uint32_t row = 16u * wave + c;
-      if (row < rows) put_pair(s, opnd, row, n0 + 4u * kg, gt, up);
+      if (row < rows) put_pair_or_tail(s, act, opnd, row, n0 + 4u * kg, gt, up);
     }
   } else if (wave < 2 * MT) {
     f4_t v = red[0][wave][lane];
     for (int w = 1; w < 8; w++) v += red[w][wave][lane];
     const uint32_t row = 16u * (wave % MT) + c;
-    if (row < rows) put_out<float>(s, act, row, n0 + 16u * (wave / MT) + 4u * kg, v);
+    if (row < rows) put_out(s, act, row, n0 + 16u * (wave / MT) + 4u * kg, v);
   }
 }
 
 // ---- tiles --------------------------------------------------------------------------------------------------------
-// BM tokens x BN matrix rows, 64 columns of K a step, four waves as 2 x 2.  Tiles go straight to LDS (16 bytes a lane,
-// eight rows of 128 bytes an instruction); chunk j of a row sits at slot j ^ (row & 7), which spreads the 16-byte reads
-// of 16 rows over the banks.  Two buffers: the next step's loads run under this step's products.
-template <int R>
-__device__ __forceinline__ void tile_load(const bf16_t* __restrict__ base, uint32_t first, uint32_t last, uint32_t kp, uint32_t k,
-                                          bf16_t* lds, uint32_t wave, uint32_t lane) {
-#pragma unroll
-  for (int i = 0; i < R / 32; i++) {
-    const uint32_t r = (uint32_t)i * 32u + wave * 8u + (lane >> 3);
-    const bf16_t* src = base + (uint64_t)min(first + r, last) * kp + k + (((lane & 7u) ^ (r & 7u)) << 3);
-    __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
-                                     (__attribute__((address_space(3))) void*)(lds + ((uint32_t)i * 32u + wave * 8u) * 64u), 16, 0, 0);
-  }
-}
 template <int BM, int BN>
 __global__ void __launch_bounds__(256)
 k_linear_tiled(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X, float* act, bf16_t* opnd, const LinSpec s, uint32_t rows,
                uint32_t tiles_m, uint32_t tiles_n) {
-  __shared__ __attribute__((aligned(16))) bf16_t la[2][BN * 64], lb[2][BM * 64];
+  __shared__ __attribute__((aligned(16))) bf16_t la[2 * BN * 64], lb[2 * BM * 64];
   constexpr int NTN = BN / 32, NTM = BM / 32;
   const uint32_t lane = threadIdx.x & 63u, wave = (uint32_t)__builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
   const uint32_t c = lane & 15u, kg = lane >> 4, kp = s.k_stride;
@@ -338,56 +400,23 @@ k_linear_tiled(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X, float
   const uint32_t m0 = (id % tiles_m) * BM, n0 = (id / tiles_m) * BN;
   const uint32_t wn = (wave & 1u) * (BN / 2), wm = (wave >> 1) * (BM / 2);
   f4_t acc[NTN][NTM];
-#pragma unroll
-  for (int i = 0; i < NTN; i++)
-#pragma unroll
-    for (int j = 0; j < NTM; j++) acc[i][j] = (f4_t){0, 0, 0, 0};
-  tile_load<BN>(W, n0, s.n - 1u, kp, 0, la[0], wave, lane);
-  tile_load<BM>(X, m0, rows - 1u, kp, 0, lb[0], wave, lane);
-  uint32_t buf = 0;
-  for (uint32_t k = 0; k < kp; k += 64u, buf ^= 1u) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();                       // this step's tiles have arrived, the other buffer is no longer read
-    if (k + 64u < kp) {
-      tile_load<BN>(W, n0, s.n - 1u, kp, k + 64u, la[buf ^ 1u], wave, lane);
-      tile_load<BM>(X, m0, rows - 1u, kp, k + 64u, lb[buf ^ 1u], wave, lane);
-    }
-#pragma unroll
-    for (int h = 0; h < 2; h++) {
-      bf8_t a[NTN], b[NTM];
-#pragma unroll
-      for (int i = 0; i < NTN; i++) {
-        const uint32_t r = wn + 16u * i + c;
-        a[i] = *(const bf8_t*)(la[buf] + r * 64u + (((4u * h + kg) ^ (r & 7u)) << 3));
-      }
-#pragma unroll
-      for (int j = 0; j < NTM; j++) {
-        const uint32_t r = wm + 16u * j + c;
-        b[j] = *(const bf8_t*)(lb[buf] + r * 64u + (((4u * h + kg) ^ (r & 7u)) << 3));
-      }
-#pragma unroll
-      for (int i = 0; i < NTN; i++)
-#pragma unroll
-        for (int j = 0; j < NTM; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[j], acc[i][j], 0, 0, 0);
-    }
-  }
+  tile_product<BM, BN>(acc, TileRows<BN>(wave, lane, [&](uint32_t r) { return W + (uint64_t)min(n0 + r, s.n - 1u) * kp; }),
+                       TileRows<BM>(wave, lane, [&](uint32_t r) { return X + (uint64_t)min(m0 + r, rows - 1u) * kp; }), kp, la, lb, wave, lane);
 #pragma unroll
   for (int j = 0; j < NTM; j++) {
     const uint32_t row = m0 + wm + 16u * j + c;
     if (row >= rows) continue;
     if (s.epi == 2u) {
 #pragma unroll
-      for (int i = 0; i < NTN; i += 2) put_pair(s, opnd, row, n0 + wn + 16u * i + 4u * kg, acc[i][j], acc[i + 1][j]);
+      for (int i = 0; i < NTN; i += 2) put_pair_or_tail(s, act, opnd, row, n0 + wn + 16u * i + 4u * kg, acc[i][j], acc[i + 1][j]);
     } else {
 #pragma unroll
-      for (int i = 0; i < NTN; i++) put_out<float>(s, act, row, n0 + wn + 16u * i + 4u * kg, acc[i][j]);
+      for (int i = 0; i < NTN; i++) put_out(s, act, row, n0 + wn + 16u * i + 4u * kg, acc[i][j]);
     }
   }
 }
 
 // ---- float32 operands ---------------------------------------------------------------------------------------------
-// 64 tokens x 64 matrix rows, 32 columns a step, on the float32 matrix instruction.  Within a run of 16 columns,
-// instruction i takes column 4 g + i from lane group g on both sides, so a lane's operands are one 16-byte read.
 __global__ void __launch_bounds__(256)
 k_linear_f32(const bf16_t* __restrict__ W, const float* __restrict__ X, float* act, float* opnd, const LinSpec s, uint32_t rows) {
   __shared__ __attribute__((aligned(16))) float la[64][36], lb[64][36];
@@ -396,40 +425,16 @@ k_linear_f32(const bf16_t* __restrict__ W, const float* __restrict__ X, float* a
   const uint32_t lr = tid >> 2, lc = (tid & 3u) * 8u;
   const bf16_t* wsrc = W + (uint64_t)min(n0 + lr, s.n - 1u) * kp + lc;
   const float* xsrc = X + (uint64_t)min(m0 + lr, rows - 1u) * kp + lc;
-  f4_t acc[2][2] = {{{0, 0, 0, 0}, {0, 0, 0, 0}}, {{0, 0, 0, 0}, {0, 0, 0, 0}}};
-  for (uint32_t k = 0; k < kp; k += 32u) {
-    const uint4 w = *(const uint4*)(wsrc + k);
-    const float4 x0 = *(const float4*)(xsrc + k), x1 = *(const float4*)(xsrc + k + 4);
-    __syncthreads();
-    *(float4*)&la[lr][lc] = make_float4(bf_lo(w.x), bf_hi(w.x), bf_lo(w.y), bf_hi(w.y));
-    *(float4*)&la[lr][lc + 4] = make_float4(bf_lo(w.z), bf_hi(w.z), bf_lo(w.w), bf_hi(w.w));
-    *(float4*)&lb[lr][lc] = x0;
-    *(float4*)&lb[lr][lc + 4] = x1;
-    __syncthreads();
-#pragma unroll
-    for (int h = 0; h < 2; h++) {
-      f4_t a[2], b[2];
-#pragma unroll
-      for (int i = 0; i < 2; i++) {
-        a[i] = *(const f4_t*)&la[wn + 16u * i + c][16u * h + 4u * kg];
-        b[i] = *(const f4_t*)&lb[wm + 16u * i + c][16u * h + 4u * kg];
-      }
-#pragma unroll
-      for (int t = 0; t < 4; t++)
-#pragma unroll
-        for (int i = 0; i < 2; i++)
-#pragma unroll
-          for (int j = 0; j < 2; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i][t], b[j][t], acc[i][j], 0, 0, 0);
-    }
-  }
+  f4_t acc[2][2];
+  tile_product_f32(acc, wsrc, xsrc, kp, la, lb);
 #pragma unroll
   for (int j = 0; j < 2; j++) {
     const uint32_t row = m0 + wm + 16u * j + c;
     if (row >= rows) continue;
-    if (s.epi == 2u) put_pair(s, opnd, row, n0 + wn + 4u * kg, acc[0][j], acc[1][j]);
+    if (s.epi == 2u) put_pair_or_tail(s, act, opnd, row, n0 + wn + 4u * kg, acc[0][j], acc[1][j]);
     else
 #pragma unroll
-      for (int i = 0; i < 2; i++) put_out<float>(s, act, row, n0 + wn + 16u * i + 4u * kg, acc[i][j]);
+      for (int i = 0; i < 2; i++) put_out(s, act, row, n0 + wn + 16u * i + 4u * kg, acc[i][j]);
   }
 }
 
@@ -449,13 +454,27 @@ static int check_linear(Map* ma, Map* mo, Map* mw, const LinSpec& s, uint32_t ro
   if (!(rows > 1 && s.ready) && !span_ok(s.src, s.src_stride, src_rows, s.k, ma->n_elems)) return ADAMAH_ERR_INVALID;
   if (s.wt_len && !in_range(s.wt, s.wt_len, ma->n_elems)) return ADAMAH_ERR_INVALID;
   if (s.gate_act && !span_ok(s.gate, s.gate_stride, src_rows, s.k, ma->n_elems)) return ADAMAH_ERR_INVALID;
-  if (s.epi == 2u && (s.n & 31u)) return ADAMAH_ERR_INVALID;
+  if (s.tail > s.n || (s.tail && s.epi != 2u) || (s.epi == 2u && ((s.n - s.tail) & 31u)) || s.gate_act > 3u) return ADAMAH_ERR_INVALID;
+  if (s.tail && !span_ok(s.tail_out, s.tail_stride, rows, s.tail, ma->n_elems)) return ADAMAH_ERR_INVALID;
+  if (s.biased && (s.epi == 2u || !in_range(s.bias, s.n, ma->n_elems))) return ADAMAH_ERR_INVALID;
+  if (!(rows > 1 && s.ready)) {
+    if (s.branched > 2u || (s.branched && (s.groups != 1u || s.gate_act || (s.wt_len && s.wt_len != s.k)))) return ADAMAH_ERR_INVALID;
+    if (s.branched && (!span_ok(s.branch, s.branch_stride, src_rows, s.k, ma->n_elems) || !in_range(s.branch_wt, s.k, ma->n_elems))) return ADAMAH_ERR_INVALID;
+    if (s.branched == 2u) {                 // workgroups read src while one of them writes the sum
+      if (!span_ok(s.res_out, s.res_stride, src_rows, s.k, ma->n_elems)) return ADAMAH_ERR_INVALID;
+      for (const auto& r : {std::make_pair(s.src, s.src_stride), std::make_pair(s.branch, s.branch_stride)}) {
+        const uint64_t e0 = s.res_out + (uint64_t)(src_rows - 1) * s.res_stride + s.k, e1 = r.first + (uint64_t)(src_rows - 1) * r.second + s.k;
+        if (s.res_out < e1 && r.first < e0) return ADAMAH_ERR_INVALID;
+      }
+    }
+    if (s.kept && !span_ok(s.keep, s.keep_stride, src_rows, s.k, ma->n_elems)) return ADAMAH_ERR_INVALID;
+  }
   if (rows > 1) {
     if (!mo || (mo->dtype != DTYPE_BF16 && mo->dtype != DTYPE_F32) || (s.opnd & 7u)) return ADAMAH_ERR_INVALID;
     if (!span_ok(s.opnd, s.k_stride, rows, s.k_stride, mo->n_elems)) return ADAMAH_ERR_INVALID;
   }
-  if (s.epi == 2u && rows > 1) return span_ok(s.out_opnd, s.out_opnd_stride, rows, s.n / 2, mo->n_elems) ? ADAMAH_OK : ADAMAH_ERR_INVALID;
-  return span_ok(s.out, s.out_stride, rows, s.epi == 2u ? s.n / 2 : s.n, ma->n_elems) ? ADAMAH_OK : ADAMAH_ERR_INVALID;
+  if (s.epi == 2u && rows > 1) return span_ok(s.out_opnd, s.out_opnd_stride, rows, (s.n - s.tail) / 2, mo->n_elems) ? ADAMAH_OK : ADAMAH_ERR_INVALID;
+  return span_ok(s.out, s.out_stride, rows, s.epi == 2u ? (s.n - s.tail) / 2 : s.n, ma->n_elems) ? ADAMAH_OK : ADAMAH_ERR_INVALID;
 }
 
 static uint32_t gemv_grid(uint32_t n_tasks) { return std::min<uint32_t>(cdiv(n_tasks, 8), 2u * (uint32_t)g.n_cu); }
@@ -477,7 +496,7 @@ static void gemv_launch(Map* ma, Map* mw, const LinSpec& s, const uint32_t* row_
 int run_linear(Map* ma, Map* mo, Map* mw, const LinSpec& s, const uint32_t* row_idx, uint32_t rows) {
   float* act = (float*)ma->buf;
   if (rows == 1) {
-    if (s.epi == 2u) gemv_launch<LEPI_PAIR>(ma, mw, s, row_idx, s.n / 2);
+    if (s.epi == 2u) gemv_launch<LEPI_PAIR>(ma, mw, s, row_idx, (s.n - s.tail) / 2 + cdiv(s.tail, 2));
     else if (s.epi == 1u) gemv_launch<LEPI_ADD>(ma, mw, s, row_idx, cdiv(s.n, 2));
     else gemv_launch<LEPI_STORE>(ma, mw, s, row_idx, cdiv(s.n, 2));
     return check_launch();
@@ -539,7 +558,7 @@ k_merge_norm(const AdamahMergeSpec s, float* act) {
   for (int w = 0; w < NT / 64; w++) { sa += sh[0][w]; sb += sh[1][w]; }
   const float ia = 1.0f / sqrtf(sa / (float)s.dim + s.eps), ib = 1.0f / sqrtf(sb / (float)s.dim + s.eps);
 #pragma unroll 4
-  for (uint32_t i = tid; i < s.dim; i += NT) d[i] += s.scale * (a[i] * ia * act[s.wa + i] + b[i] * ib * act[s.wb + i]);
+  for (uint32_t i = tid; i < s.dim; i += NT) d[i] = (s.store ? 0.f : d[i]) + s.scale * (a[i] * ia * act[s.wa + i] + b[i] * ib * act[s.wb + i]);
 }
 
 }  // namespace adamah

@@ -408,8 +408,10 @@ void adamah_shutdown(void) { ADAMAH_API();
   attn_prefill_release();
   token_feed_release();
   linear_release();
+  state_space_release();
+  experts_release();
   recurrent_release();
-  attn_chunk_release();
+  attn_bounded_release();
   g.pend.clear();
   for (int i = 0; i < MAX_PLANS; i++) { g.plans[i].clear(); g.plan_active[i] = false; plan_graph_reset(i); }
   hipStreamDestroy(g.stream);
@@ -859,6 +861,9 @@ static int replay_plan(uint32_t plan_id, uint32_t pos, uint32_t seq_len) {
       case 34: ret = adamah_delta_rule_dev(op.map_id, op.op_code, op.map_id2, op.h0, op.h1, op.h2, u0, u1, u2, u3); break;
       case 35: ret = adamah_retention_dev(op.map_id, op.h0, u0, u1, u2, u3); break;
       case 36: ret = adamah_chunk_attention_dev(op.map_id, op.h0, u0, u1, u2, u3); break;
+      case 37: ret = adamah_window_attention_dev(op.map_id, op.h0, u0, u1, u2, u3); break;
+      case 38: ret = adamah_state_space_dev(op.map_id, op.h0, u0, u1, u2, u3); break;
+      case 39: ret = adamah_experts_dev(op.map_id, op.op_code, op.map_id2, op.h0, op.h1, u0); break;
       default: ret = ADAMAH_ERR_INVALID; break;
     }
     if (ret != ADAMAH_OK) break;

@@ -68,6 +68,40 @@ k_embed_tokens(float* act, uint64_t act_elems, const uint8_t* __restrict__ src, 
   act[dst0 + i] = v;
 }
 
+// One workgroup per row: scale * row of the token table + row of the bigram table (AdamahBigramSpec).  The workgroup that
+// starts a sequence's rows is the only one to touch its previous token in the state map: it reads it and then leaves the
+// last row's token there.
+template <bool BF>
+__global__ void __launch_bounds__(512)
+k_embed_bigram(const AdamahBigramSpec s, float* act, uint64_t act_elems, const uint8_t* __restrict__ src, const uint32_t* __restrict__ tok_locs,
+               float* state, uint32_t rows, uint32_t seq0, uint32_t pos, TokenMail* mail, uint32_t ticket, uint32_t n_tok) {
+  if (mail && blockIdx.x == 0 && threadIdx.x < 64u) {
+    if (threadIdx.x < n_tok) mail->val[threadIdx.x] = tok_locs[threadIdx.x] < act_elems ? act[tok_locs[threadIdx.x]] : 0.0f;
+    __threadfence_system();
+    if (threadIdx.x == 0) {
+      mail->n = n_tok;
+      __hip_atomic_store(&mail->ticket, ticket, __ATOMIC_RELEASE, __HIP_MEMORY_SCOPE_SYSTEM);
+    }
+  }
+  const uint32_t r = blockIdx.x, seq = r / rows, t = r - seq * rows;       // rows tokens of each sequence
+  float* kept = state + (uint64_t)(seq0 + seq) * s.seq_stride + s.prev_off;
+  const auto token = [&](uint32_t i) { const uint32_t l = tok_locs[i]; return l < act_elems ? act[l] : -1.0f; };
+  const float tf = token(r), pf = t ? token(r - 1u) : pos ? *kept : 0.0f;
+  const bool ok = tf >= 0.0f && tf < (float)s.vocab && pf >= 0.0f && pf < 4294967040.0f;
+  const uint64_t tok = ok ? (uint32_t)tf : 0u, prev = ok ? (uint32_t)pf : 0u;
+  const uint64_t pair = pos + t == 0u ? s.buckets : (prev * s.mul_prev + tok * s.mul_cur) % s.buckets;
+  const uint64_t a = s.table + tok * s.width, b = s.pairs + pair * s.width;
+  for (uint32_t i = threadIdx.x; i < s.width; i += 512u) {
+    float v = 0.0f;
+    if (ok) v = BF ? fmaf(__uint_as_float((uint32_t)((const uint16_t*)src)[a + i] << 16), s.scale, __uint_as_float((uint32_t)((const uint16_t*)src)[b + i] << 16))
+                   : fmaf(((const float*)src)[a + i], s.scale, ((const float*)src)[b + i]);
+    act[s.dst + (uint64_t)r * s.width + i] = v;
+  }
+  if (t) return;
+  __syncthreads();                                                         // every thread has the previous token
+  if (threadIdx.x == 0) *kept = token(r + rows - 1u);
+}
+
 // One wave: values first, then the ticket, both for the host (system scope).
 __global__ void __launch_bounds__(64)
 k_token_post(const float* __restrict__ act, uint64_t act_elems, const uint32_t* __restrict__ locs, uint32_t n,
@@ -159,6 +193,37 @@ int adamah_hip_embed_post_tokens_dev(uint32_t map_act, uint32_t map_src, uint32_
                                      uint32_t* ticket) { ADAMAH_API();
   if (!ticket) return ADAMAH_ERR_INVALID;
   return embed_tokens(map_act, map_src, locs_tokens, src_row0, dst_start, m, E, V, scale, ticket);
+}
+
+int adamah_hip_embed_bigram_dev(uint32_t map_act, uint32_t map_src, uint32_t h_spec, uint32_t locs_tokens, uint32_t n_seq,
+                                uint32_t rows, uint32_t seq0, uint32_t pos, uint32_t* ticket_out) { ADAMAH_API();
+  Map *ma = get_f32_map(map_act), *ms = get_map(map_src);
+  const AdamahBigramSpec* s = (const AdamahBigramSpec*)res_host(h_spec, sizeof(AdamahBigramSpec) / 4);
+  if (!ma || !ms || !s || n_seq == 0 || rows == 0 || (n_seq > 1 && rows > 1) || ms->pack_size != 1 || ma->pack_size != 1) return ADAMAH_ERR_INVALID;
+  if (ms->dtype != DTYPE_BF16 && ms->dtype != DTYPE_F32) return ADAMAH_ERR_INVALID;
+  Map* mt = get_f32_map(s->state_map);
+  const uint64_t m = (uint64_t)n_seq * rows;
+  if (!mt || s->vocab == 0 || s->width == 0 || s->buckets == 0 || s->prev_off >= s->seq_stride || m > 0x7FFFFFFFull) return ADAMAH_ERR_INVALID;
+  if (!in_range((uint64_t)seq0 * s->seq_stride, (uint64_t)n_seq * s->seq_stride, mt->n_elems) || !in_range(s->dst, m * s->width, ma->n_elems) ||
+      !in_range(s->table, (uint64_t)s->vocab * s->width, ms->n_elems) ||
+      !in_range(s->pairs, ((uint64_t)s->buckets + 1) * s->width, ms->n_elems)) return ADAMAH_ERR_INVALID;
+  if (ma->kv16 && s->dst < ma->kv_start + ma->kv_count && ma->kv_start < s->dst + m * s->width) return ADAMAH_ERR_INVALID;
+  const uint32_t* tl = res_u32(locs_tokens, m);
+  if (!tl) return ADAMAH_ERR_INVALID;
+  TokenMail* mail = nullptr;
+  uint32_t ticket = 0;
+  if (ticket_out) {
+    if (m > MAIL_MAX) return ADAMAH_ERR_INVALID;
+    if (int r = mail_setup()) return r;
+    ticket = g_ticket = g_ticket >= 0x7FFFFFFFu ? 1u : g_ticket + 1u;
+    *ticket_out = ticket;
+    mail = g_mail_dev + ticket % MAIL_SLOTS;
+  }
+#define EMBED(BF) k_embed_bigram<BF><<<(uint32_t)m, 512, 0, g.stream>>>(*s, (float*)ma->buf, ma->n_elems, ms->buf, tl, (float*)mt->buf, rows, seq0,                                                                       pos, mail, ticket, (uint32_t)m)
+  if (ms->dtype == DTYPE_BF16) EMBED(true); else EMBED(false);
+#undef EMBED
+  count_launch();
+  return check_launch();
 }
 
 int adamah_hip_token_post(uint32_t map_id, uint32_t locs_handle, uint32_t n, uint32_t* ticket_out) { ADAMAH_API();

@@ -681,7 +681,7 @@ class DecodeEngine:
                 row = row * np.float32(c.emb_scale)
             g.scatter(self.WS_MAP, self._hid_locs, row)
 
-    def _issue_embedding(self, from_device):
+    def _issue_embedding(self, from_device, pos):
         c, g, A, ws, W = self.cfg, self.gpu, self.A, self.WS_MAP, self._ws
         hid_h = W['hidden'][0]
         if from_device:     # (the same launch hands the token to the host: _wait_tokens(self._feed_ticket))
@@ -777,7 +777,7 @@ class DecodeEngine:
         normed_h = W['normed'][0]
         self._stage_token(tok, from_device)
         g.batch_begin()
-        self._issue_embedding(from_device)
+        self._issue_embedding(from_device, pos)
         self._issue_layers(pos)
         if from_device and on_token is not None and not on_token(self._wait_tokens(self._feed_ticket)[0]):
             g.batch_end()

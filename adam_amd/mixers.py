@@ -9,6 +9,7 @@ Another mixer is another class with these members:
   tensors(E)            name -> shape, None where the tensor decides
   inputs()              names of the stacked input projections, in order
   vectors()             names of the tensors kept as float32 in the workspace
+  biases()              names of the stacked input projections' biases, in the inputs' order ([]: none)
   widths(shape)         row buffer -> width it needs
   state_size(), cache_size()   elements per sequence in the float32 state map / in the key-value cache map
   const_size()          float32 constants from the configuration (`e.const`)
@@ -35,8 +36,13 @@ def _grouped(name, heads, kv_heads):
         raise ValueError(f"{name}: {heads} heads do not share {kv_heads} key heads evenly")
 
 
+class Mixer:
+    def biases(self):
+        return []
+
+
 @dataclass
-class ChannelDelta:
+class ChannelDelta(Mixer):
     """Gated delta rule: short convolutions on q, k, v, unit q and k, one decay per head and key channel (low-rank),
     per-head norm and a low-rank sigmoid gate on the way out."""
     heads: int
@@ -101,7 +107,7 @@ class ChannelDelta:
 
 
 @dataclass
-class ChunkAttention:
+class ChunkAttention(Mixer):
     """Softmax attention over the keys of the query's own chunk, with r1 ln(1 + r2 distance) taken off the scores and
     values divided by their root mean square; grouped key / value heads, no rotation."""
     heads: int
@@ -162,7 +168,7 @@ class ChunkAttention:
 
 
 @dataclass
-class Retention:
+class Retention(Mixer):
     """Linear attention with one fixed decay per head; rotary q and k, per-head norm without weight, silu gate."""
     heads: int
     dim: int
@@ -222,7 +228,7 @@ class Retention:
 
 
 @dataclass
-class Parallel:
+class Parallel(Mixer):
     """Mean of two branches over the same input, each through a full-width RMS norm with a weight of its own."""
     left: object
     right: object
@@ -270,10 +276,148 @@ class Parallel:
             m.core(e, p + n, self._cols(x, n))
 
     def output(self, e, p, x, out, epi):
-        assert epi == e.A.EPI_ADD
         for (n, m), rows in zip(self._both(), ("y", "y2")):
             m.output(e, p + n, self._cols(x, n), e.at(rows), e.A.EPI_STORE)
-        e.merge("y", "y2", e.vec(p + "left.out"), e.vec(p + "right.out"), out, 0.5)
+        e.merge("y", "y2", e.vec(p + "left.out"), e.vec(p + "right.out"), out, 0.5, epi)
 
 
-MIXERS = {"channel_delta": ChannelDelta, "parallel": Parallel}
+@dataclass
+class WindowAttention(Mixer):
+    """Softmax attention over a sliding window with a learned sink per head in the denominator: queries and keys divided by
+    their root mean square, a query temperature that grows with the logarithm of the position, capped scores, a linear
+    distance penalty per head; grouped key / value heads, biased projections, no rotation."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int
+    softcap: float = 0.0
+    temp_coef: float = 0.0
+    temp_every: int = 1
+    rows: str = "o"
+
+    @classmethod
+    def from_config(cls, d, rows="o"):
+        t = d.get("q_temp") or {}
+        return cls(int(d["heads"]), int(d["kv_heads"]), int(d["dim"]), int(d["vdim"]), float(d["scale"]), int(d["mask"]["size"]),
+                   float(d.get("softcap") or 0.0), float(t.get("coef", 0.0)), int(t.get("every", 1)), rows)
+
+    def __post_init__(self):
+        _fits("window attention", dim=self.dim, vdim=self.vdim)
+        _grouped("window attention", self.heads, self.kv_heads)
+        if self.window < 1 or self.softcap < 0 or self.temp_every < 1:
+            raise ValueError(f"window attention: window {self.window}, cap {self.softcap}, temperature every {self.temp_every}")
+
+    def tensors(self, E):
+        H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
+        return {"q": (H * D, E), "q.b": (H * D,), "k": (G * D, E), "k.b": (G * D,), "v": (G * V, E), "v.b": (G * V,), "sink": (H,),
+                "o": (E, H * V)}
+
+    def inputs(self):
+        return ["q", "k", "v"]
+
+    def biases(self):
+        return ["q.b", "k.b", "v.b"]
+
+    def vectors(self):
+        return ["sink"]
+
+    def widths(self, shape):
+        return {self.rows: self.heads * self.vdim}
+
+    def state_size(self):
+        return 0
+
+    def cache_size(self):
+        r8 = lambda n: (n + 7) // 8 * 8
+        return self.kv_heads * self.window * (r8(self.dim) + r8(self.vdim))
+
+    def const_size(self):
+        return self.heads
+
+    def core(self, e, p, x):
+        r8 = lambda n: (n + 7) // 8 * 8
+        off = e.take_cache(self.cache_size())
+        xo, xs = e.at("x")
+        oo, os_ = e.at(self.rows)
+        slope = e.const(2.0 ** (-8.0 * np.arange(1, self.heads + 1) / self.heads))
+        e.window_attention(e.A.WindowAttnSpec(
+            heads=self.heads, kv_heads=self.kv_heads, dim=self.dim, vdim=self.vdim, window=self.window, x=xo, x_stride=xs,
+            x_q=x["q"], x_k=x["k"], x_v=x["v"], slope=slope, sink=e.vec(p + "sink"), has_sink=1, qk_norm=1, scale=self.scale,
+            eps=e.cfg.norm_eps, softcap=self.softcap, temp_coef=self.temp_coef, temp_every=self.temp_every, out=oo, out_stride=os_,
+            cache_map=e.CACHE_MAP, k_off=off, v_off=off + self.kv_heads * self.window * r8(self.dim), seq_stride=e.cache_per_seq))
+
+    def output(self, e, p, x, out, epi):
+        e.linear([p + "o"], src=e.at(self.rows), out=out, epi=epi)
+
+
+@dataclass
+class StateSpace(Mixer):
+    """Mamba-2: one projection for gate, inputs and step sizes, a short biased convolution, a state per head that decays by
+    one factor per token, gate ahead of a norm in equal parts."""
+    heads: int
+    groups: int
+    state: int
+    vdim: int
+    conv: int
+    norm_groups: int
+
+    @classmethod
+    def from_config(cls, d):
+        return cls(*(int(d[n]) for n in ("heads", "groups", "state", "vdim", "conv", "norm_groups")))
+
+    def __post_init__(self):
+        _fits("state space", state=self.state, vdim=self.vdim, conv=self.conv)
+        if self.groups < 1 or self.heads % self.groups:
+            raise ValueError(f"state space: {self.heads} heads do not share {self.groups} groups evenly")
+        if self.norm_groups < 1 or self.inner % self.norm_groups:
+            raise ValueError(f"state space: {self.inner} channels do not split into {self.norm_groups} norm groups")
+
+    @property
+    def inner(self):
+        return self.heads * self.vdim
+
+    @property
+    def channels(self):
+        return self.inner + 2 * self.groups * self.state
+
+    def tensors(self, E):
+        return {"in": (self.inner + self.channels + self.heads, E), "conv": (self.channels, self.conv), "conv.b": (self.channels,),
+                "dt_bias": (self.heads,), "A_log": (self.heads,), "D": (self.heads,), "norm": (self.inner,), "o": (E, self.inner)}
+
+    def inputs(self):
+        return ["in"]
+
+    def vectors(self):
+        return ["conv", "conv.b", "dt_bias", "A_log", "D", "norm"]
+
+    def widths(self, shape):
+        return {"o": self.inner}
+
+    def state_size(self):
+        return self.heads * self.state * self.vdim + self.conv * self.channels
+
+    def cache_size(self):
+        return 0
+
+    def const_size(self):
+        return 0
+
+    def core(self, e, p, x):
+        xo, xs = e.at("x", x["in"])
+        oo, os_ = e.at("o")
+        s_off = e.take_state(self.state_size())
+        e.state_space(e.A.StateSpaceSpec(
+            heads=self.heads, groups=self.groups, state=self.state, vdim=self.vdim, taps=self.conv, x=xo, x_stride=xs, x_c=self.inner,
+            x_dt=self.inner + self.channels, conv=e.vec(p + "conv"), conv_b=e.vec(p + "conv.b"), dt_bias=e.vec(p + "dt_bias"),
+            a_log=e.vec(p + "A_log"), skip=e.vec(p + "D"), out=oo, out_stride=os_, state_map=e.STATE_MAP, s_off=s_off,
+            conv_off=s_off + self.heads * self.state * self.vdim, seq_stride=e.state_per_seq))
+
+    def output(self, e, p, x, out, epi):
+        zo, zs = e.at("x", x["in"])
+        e.linear([p + "o"], src=e.at("o"), out=out, epi=epi,
+                 norm=e.norm(self.norm_groups, e.vec(p + "norm"), self.inner, gate=(zo, zs, e.A.GATE_SILU_AHEAD)))
+
+
+MIXERS = {"channel_delta": ChannelDelta, "parallel": Parallel, "attention": WindowAttention, "mamba2": StateSpace}

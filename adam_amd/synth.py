@@ -130,6 +130,7 @@ def make_model(cfg, seed=0, sigma=0.02, workers=None):
 def mixer_config(width, ff, heads, head_dim, kv_heads, n_layer=4, n_vocab=32768, chunk=8192):
     """A layered mixer model with the proportions of a real one: three delta-rule layers to one parallel layer (chunk
     attention with grouped heads beside retention), head sizes of 128."""
+    from .feed_forward import Dense
     from .mixers import ChannelDelta, ChunkAttention, Parallel, Retention
     from .models import MixerConfig, MixerLayer
     layers = []
@@ -140,7 +141,7 @@ def mixer_config(width, ff, heads, head_dim, kv_heads, n_layer=4, n_vocab=32768,
             decay = tuple(1.0 - 2.0 ** -(5 + 7 * h / max(heads - 1, 1)) for h in range(heads))
             m = Parallel(ChunkAttention(heads, kv_heads, head_dim, head_dim, head_dim ** -0.5, chunk, "o"),
                          Retention(heads, head_dim, head_dim, decay, 1e4, head_dim, "o2"))
-        layers.append(MixerLayer(m, ff))
+        layers.append(MixerLayer(m, Dense(ff)))
     return MixerConfig(arch="Vomotar", n_vocab=n_vocab, n_embd=width, norm_groups=4, norm_eps=1e-6, layers=layers)
 
 

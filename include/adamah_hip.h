@@ -287,28 +287,36 @@ int adamah_hip_token_wait(uint32_t ticket, float* out, uint32_t n);
  * element offsets: into the float32 activation map unless said otherwise.  "Rows" are tokens; their buffers are
  * row-major with the stride the spec names. */
 
-/* y = W . f(x) for `rows` rows, W [n, k] in a bfloat16 map, its rows k_stride apart (a multiple of 64, zeros beyond k).
- * f: groups = 0: nothing.  Else the row is cut into `groups` equal runs, each divided by sqrt(mean of squares + eps),
- * then multiplied by the weight (wt_len = 0: none; wt_len < k: repeated) and by the gate (gate_act 1: sigmoid, 2: silu,
- * of the element at gate + row * gate_stride).  Rows > 1 go through the operand map (bfloat16: bfloat16 matrix
- * instructions, float32: float32 ones) at `opnd`, rows k_stride apart; ready = 1: they are there already.
+/* y = W . f(x) (+ bias) for `rows` rows, W [n, k] in a bfloat16 map, its rows k_stride apart (a multiple of 64, zeros
+ * beyond k).  f: groups = 0: nothing.  Else the row is cut into `groups` equal runs, each divided by sqrt(mean of squares
+ * + eps), then multiplied by wt_add + the weight (wt_len = 0: none; wt_len < k: repeated) and by the gate (gate_act 1:
+ * sigmoid, 2: silu, of the element at gate + row * gate_stride).  gate_act 3: silu, multiplied in ahead of the norm.
+ * branched (groups = 1): what is normed is the row of src plus the row of `branch` after a norm of its own, over its full
+ * width, times wt_add + branch_wt; branched = 2: that sum is also stored at res_out (which src must not overlap).
+ * kept = 1: f(x) is also stored, as float32, at `keep`.  biased = 1: bias[n] is added.
+ * Rows > 1 go through the operand map (bfloat16: bfloat16 matrix instructions, float32: float32 ones) at `opnd`, rows
+ * k_stride apart; ready = 1: they are there already.
  * epi 0: out = y.  1: out += y.  2: W holds 16 gate rows, their 16 up rows, and so on; silu(gate) * up goes to `out`
- * (one row) or to the operand map at out_opnd (more rows), n / 2 columns. */
+ * (one row) or to the operand map at out_opnd (more rows), (n - tail) / 2 columns.  The last `tail` rows (epi 2) are
+ * ordinary ones: their y goes to tail_out. */
 typedef struct AdamahLinearSpec {
   uint32_t w, n, k, k_stride, src, src_stride, groups;
   float eps;
   uint32_t wt, wt_len, gate, gate_stride, gate_act, opnd, ready, out, out_stride, epi, out_opnd, out_opnd_stride;
+  float wt_add;
+  uint32_t bias, biased, branch, branch_stride, branch_wt, branched, res_out, res_stride, keep, keep_stride, kept;
+  uint32_t tail, tail_out, tail_stride;
 } AdamahLinearSpec;
 /* h_rows: 0, or a handle that names the source row of each row. */
 int adamah_linear_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, uint32_t h_spec, uint32_t h_rows, uint32_t rows);
 /* The same (epi 0), then float(arg-max of row r) to element dst[r] of the activation map (h_dst: `rows` offsets). */
 int adamah_linear_argmax_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, uint32_t h_spec, uint32_t h_dst, uint32_t rows);
 
-/* dst += scale * (a / rms(a) * wa + b / rms(b) * wb) per row. */
-typedef struct AdamahMergeSpec { uint32_t a, b, stride, wa, wb, dst, dst_stride, dim; float eps, scale; } AdamahMergeSpec;
+/* dst += scale * (a / rms(a) * wa + b / rms(b) * wb) per row (store = 1: dst =). */
+typedef struct AdamahMergeSpec { uint32_t a, b, stride, wa, wb, dst, dst_stride, dim; float eps, scale; uint32_t store; } AdamahMergeSpec;
 int adamah_merge_norm_dev(uint32_t map_act, uint32_t h_spec, uint32_t rows);
 
-/* The three sequence mixers below take `rows` consecutive tokens of one sequence (n_seq = 1, slot seq0) at positions
+/* The sequence mixers below take `rows` consecutive tokens of one sequence (n_seq = 1, slot seq0) at positions
  * pos .. pos + rows - 1, or one token of each of n_seq sequences (slots seq0 .. seq0 + n_seq - 1), all at position pos.
  * x: the rows' projections, [rows, x_stride].  State lives in a map of its own, slot s at s * seq_stride; a sequence
  * that starts (pos = 0) does not read it, so a slot can be handed to another sequence as it is. */
@@ -343,6 +351,55 @@ typedef struct AdamahChunkAttnSpec {
   uint32_t out, out_stride, cache_map, k_off, v_off, seq_stride;
 } AdamahChunkAttnSpec;
 int adamah_chunk_attention_dev(uint32_t map_act, uint32_t h_spec, uint32_t n_seq, uint32_t rows, uint32_t seq0, uint32_t pos);
+
+/* Softmax attention over a sliding window: position i sees the `window` positions i - window + 1 .. i.  qk_norm = 1: q and
+ * k are divided by their root mean square first (eps inside).  q is multiplied by 1 + temp_coef * ln(floor((i + 1) /
+ * temp_every) + 1) (temp_coef = 0: not).  score = (q . k) * scale, softcap > 0: softcap * tanh(score / softcap), then
+ * slope_h * distance is taken off.  has_sink = 1: the denominator also holds exp(sink_h).  The cache is laid out as the
+ * chunk attention's, `window` places per slot, token at place position % window; keys are cached normed. */
+typedef struct AdamahWindowAttnSpec {
+  uint32_t heads, kv_heads, dim, vdim, window, x, x_stride, x_q, x_k, x_v, slope, sink, has_sink, qk_norm;
+  float scale, eps, softcap, temp_coef;
+  uint32_t temp_every, out, out_stride, cache_map, k_off, v_off, seq_stride;
+} AdamahWindowAttnSpec;
+int adamah_window_attention_dev(uint32_t map_act, uint32_t h_spec, uint32_t n_seq, uint32_t rows, uint32_t seq0, uint32_t pos);
+
+/* State-space recurrence with one decay per head and token: dt = softplus(dt + dt_bias), S = exp(-exp(A_log) dt) S +
+ * dt B x^T, o = S^T C + D x, S [state, vdim] per head, B and C shared by heads / groups heads.  x row: at x_c the channels
+ * x [heads, vdim], B, C [groups, state] ahead of their convolution (`taps` taps, bias conv_b per channel) and silu, at x_dt
+ * the heads' step sizes.  conv: [channels, taps].  skip: D. */
+typedef struct AdamahStateSpaceSpec {
+  uint32_t heads, groups, state, vdim, taps, x, x_stride, x_c, x_dt, conv, conv_b, dt_bias, a_log, skip, out, out_stride;
+  uint32_t state_map, s_off, conv_off, seq_stride;
+} AdamahStateSpaceSpec;
+int adamah_state_space_dev(uint32_t map_act, uint32_t h_spec, uint32_t n_seq, uint32_t rows, uint32_t seq0, uint32_t pos);
+
+/* Mixture of experts over rows whose router logits are known.  A row's scores are the softmax of its `experts + identity`
+ * logits; the `top` (<= 64) with the largest score + correction are chosen, weighted by their scores as they are.  Expert
+ * e < experts: gate and up rows alternating in runs of 16 at gate_up + e * gate_up_step ([2 * ff rounded up to 16,
+ * k_stride]), W_down [width, ff_stride] at down + e * down_step; those past it give the row itself back.  The row: float32
+ * at x, and (rows > 1) at opnd in the operand map, k_stride apart.  act: ff_stride * top elements (one row); act_opnd: rows
+ * * top rows of ff_stride in the operand map.  shared_ff > 0: the shared expert's activation, at shared_act (one row),
+ * passes through W [width, shared_ff_stride] at shared_down, is multiplied by the sigmoid of logit experts + identity, and
+ * added; h_shared is the same product as a linear op (epi 0), used for more rows.  epi 0: out = y, 1: out += y. */
+typedef struct AdamahExpertsSpec {
+  uint32_t experts, identity, top, ff, ff_stride, width, k_stride, gate_up, gate_up_step, down, down_step, logits, logits_stride;
+  uint32_t correction, x, x_stride, opnd, act, act_opnd, shared_ff, shared_ff_stride, shared_down, shared_act, out, out_stride, epi;
+} AdamahExpertsSpec;
+int adamah_experts_dev(uint32_t map_act, uint32_t map_opnd, uint32_t map_wt, uint32_t h_spec, uint32_t h_shared, uint32_t rows);
+
+/* Token embedding with a bigram table: row r of dst (width apart) = scale * row tok_r of the table [vocab, width] at
+ * `table` + row (prev * mul_prev + tok_r * mul_cur) mod buckets of the table at `pairs`; a sequence's first token takes row
+ * `buckets`.  The token ahead of row r is row r - 1's, the token ahead of the first one is kept in the state map (one
+ * element per slot, at prev_off).  Tables: bfloat16 or float32 map.  ticket: NULL, or as adamah_hip_embed_post_tokens_dev.
+ * Tokens: float32 ids at the elements locs_tokens names. */
+typedef struct AdamahBigramSpec {
+  uint32_t table, vocab, width, dst;
+  float scale;
+  uint32_t pairs, buckets, mul_prev, mul_cur, state_map, prev_off, seq_stride;
+} AdamahBigramSpec;
+int adamah_hip_embed_bigram_dev(uint32_t map_act, uint32_t map_src, uint32_t h_spec, uint32_t locs_tokens, uint32_t n_seq,
+                                uint32_t rows, uint32_t seq0, uint32_t pos, uint32_t* ticket);
 
 /* ---- measurement and test helpers: not part of the op surface ------------------------------------
  * Nothing a model engine calls.  bench.py times launches with the stopwatch and calibrates profiler counters

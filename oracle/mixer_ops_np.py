@@ -8,14 +8,22 @@ import numpy as np
 
 F = np.float64
 _LINEAR = ("w n k k_stride src src_stride groups eps wt wt_len gate gate_stride gate_act opnd ready out out_stride epi "
-           "out_opnd out_opnd_stride")
-_MERGE = "a b stride wa wb dst dst_stride dim eps scale"
+           "out_opnd out_opnd_stride wt_add bias biased branch branch_stride branch_wt branched res_out res_stride keep keep_stride "
+           "kept tail tail_out tail_stride")
+_MERGE = "a b stride wa wb dst dst_stride dim eps scale store"
 _DELTA = ("heads kv_heads dim vdim taps x x_stride x_b cq ck cv a_log dt_bias out out_stride state_map s_off conv_off "
           "seq_stride")
 _RET = "heads dim vdim rot_dims freq decay x x_stride x_q x_k x_v out out_stride state_map s_off seq_stride"
 _ATT = ("heads kv_heads dim vdim chunk x x_stride x_q x_k x_v r1 r2 scale eps out out_stride cache_map k_off v_off "
         "seq_stride")
-_FLOATS = {"eps", "scale"}
+_WIN = ("heads kv_heads dim vdim window x x_stride x_q x_k x_v slope sink has_sink qk_norm scale eps softcap temp_coef temp_every "
+        "out out_stride cache_map k_off v_off seq_stride")
+_SSM = ("heads groups state vdim taps x x_stride x_c x_dt conv conv_b dt_bias a_log skip out out_stride state_map s_off conv_off "
+        "seq_stride")
+_MOE = ("experts identity top ff ff_stride width k_stride gate_up gate_up_step down down_step logits logits_stride correction x "
+        "x_stride opnd act act_opnd shared_ff shared_ff_stride shared_down shared_act out out_stride epi")
+_BIGRAM = "table vocab width dst scale pairs buckets mul_prev mul_cur state_map prev_off seq_stride"
+_FLOATS = {"eps", "scale", "wt_add", "softcap", "temp_coef"}
 
 
 class _S:
@@ -69,19 +77,32 @@ class MixerOps:
                 x = self._get(map_opnd, s.opnd + r * s.k_stride, s.k)
             else:
                 x = self._get(map_act, s.src + i * s.src_stride, s.k)
+                if s.branched:
+                    b = self._get(map_act, s.branch + i * s.branch_stride, s.k)
+                    x = x + b / np.sqrt(np.mean(b * b) + s.eps) * (s.wt_add + self._get(map_act, s.branch_wt, s.k))
+                    if s.branched == 2:
+                        self._put(map_act, s.res_out + i * s.res_stride, x)
                 if s.groups:
+                    if s.gate_act == 3:
+                        x = x * _silu(self._get(map_act, s.gate + i * s.gate_stride, s.k))
                     y = x.reshape(s.groups, -1)
                     x = (y / np.sqrt(np.mean(y * y, axis=1, keepdims=True) + s.eps)).reshape(-1)
                     if s.wt_len:
-                        x = x * np.resize(self._get(map_act, s.wt, s.wt_len), s.k)
-                    if s.gate_act:
+                        x = x * np.resize(s.wt_add + self._get(map_act, s.wt, s.wt_len), s.k)
+                    if s.gate_act in (1, 2):
                         x = x * (_sig, _silu)[s.gate_act - 1](self._get(map_act, s.gate + i * s.gate_stride, s.k))
+                if s.kept:
+                    self._put(map_act, s.keep + i * s.keep_stride, x)
                 if rows > 1:
                     self._put(map_opnd, s.opnd + r * s.k_stride, x)
                     x = self._get(map_opnd, s.opnd + r * s.k_stride, s.k)
             y = W[:, :s.k] @ x
+            if s.biased:
+                y = y + self._get(map_act, s.bias, s.n)
             if s.epi == 2:
-                y = y.reshape(-1, 2, 16)
+                if s.tail:
+                    self._put(map_act, s.tail_out + r * s.tail_stride, y[s.n - s.tail:])
+                y = y[:s.n - s.tail].reshape(-1, 2, 16)
                 y = (_silu(y[:, 0]) * y[:, 1]).reshape(-1)
                 if rows > 1:
                     self._put(map_opnd, s.out_opnd + r * s.out_opnd_stride, y)
@@ -103,7 +124,7 @@ class MixerOps:
                 x = self._get(map_act, src + r * s.stride, s.dim)
                 y = y + x / np.sqrt(np.mean(x * x) + s.eps) * self._get(map_act, w, s.dim)
             d = s.dst + r * s.dst_stride
-            self._put(map_act, d, self._get(map_act, d, s.dim) + s.scale * y)
+            self._put(map_act, d, (0.0 if s.store else self._get(map_act, d, s.dim)) + s.scale * y)
 
     @staticmethod
     def _tokens(n_seq, rows, seq0, pos):
@@ -185,3 +206,103 @@ class MixerOps:
                 sc = (K @ x[s.x_q + hd * D:s.x_q + (hd + 1) * D]) * s.scale - r1[hd] * np.log1p(r2[hd] * np.arange(n - 1, -1, -1))
                 w = np.exp(sc - sc.max())
                 self._put(map_act, s.out + r * s.out_stride + hd * V, (w / w.sum()) @ Vc)
+
+    def window_attention_dev(self, map_act, h, n_seq, rows, seq0, pos):
+        s = self._spec(h, _WIN)
+        H, G, D, V, R = s.heads, s.kv_heads, s.dim, s.vdim, s.window
+        D8, V8 = (D + 7) // 8 * 8, (V + 7) // 8 * 8
+        slope = self._get(map_act, s.slope, H)
+        rms = lambda a: a / np.sqrt(np.mean(a * a, axis=-1, keepdims=True) + s.eps) if s.qk_norm else a
+        for r, slot, p in self._tokens(n_seq, rows, seq0, pos):
+            base = slot * s.seq_stride
+            x = self._get(map_act, s.x + r * s.x_stride, s.x_stride)
+            k = rms(x[s.x_k:s.x_k + G * D].reshape(G, D))
+            q = rms(x[s.x_q:s.x_q + H * D].reshape(H, D))
+            if s.temp_coef:
+                q = q * (1.0 + s.temp_coef * np.log((p + 1) // s.temp_every + 1))
+            seen = np.arange(max(0, p - R + 1), p + 1)
+            for g in range(G):
+                k8, v8 = np.zeros(D8), np.zeros(V8)
+                k8[:D], v8[:V] = k[g], x[s.x_v + g * V:s.x_v + (g + 1) * V]
+                self._put(s.cache_map, base + s.k_off + (g * R + p % R) * D8, k8)
+                self._put(s.cache_map, base + s.v_off + (g * R + p % R) * V8, v8)
+            for hd in range(H):
+                g = hd // (H // G)
+                K = self._get(s.cache_map, base + s.k_off + g * R * D8, R * D8).reshape(R, D8)[seen % R, :D]
+                Vc = self._get(s.cache_map, base + s.v_off + g * R * V8, R * V8).reshape(R, V8)[seen % R, :V]
+                sc = (K @ q[hd]) * s.scale
+                if s.softcap:
+                    sc = s.softcap * np.tanh(sc / s.softcap)
+                sc = sc - slope[hd] * (p - seen)
+                sink = self._get(map_act, s.sink + hd, 1)[0] if s.has_sink else -np.inf
+                top = max(sc.max(), sink)
+                w = np.exp(sc - top)
+                self._put(map_act, s.out + r * s.out_stride + hd * V, (w / (w.sum() + np.exp(sink - top))) @ Vc)
+
+    def state_space_dev(self, map_act, h, n_seq, rows, seq0, pos):
+        s = self._spec(h, _SSM)
+        H, G, N, V, J = s.heads, s.groups, s.state, s.vdim, s.taps
+        n_ch = H * V + 2 * G * N
+        w, b = self._get(map_act, s.conv, n_ch * J).reshape(n_ch, J), self._get(map_act, s.conv_b, n_ch)
+        pick = np.arange(H) // (H // G)
+        for r, slot, p in self._tokens(n_seq, rows, seq0, pos):
+            base = slot * s.seq_stride
+            x = self._get(map_act, s.x + r * s.x_stride, s.x_stride)
+            ring = self._get(s.state_map, base + s.conv_off, J * n_ch).reshape(J, n_ch)
+            ring[p % J] = x[s.x_c:s.x_c + n_ch]
+            self._put(s.state_map, base + s.conv_off, ring)
+            z = _silu(b + sum(w[:, J - 1 - j] * ring[(p - j) % J] for j in range(J) if j <= p))
+            u = z[:H * V].reshape(H, V)
+            B, C = (z[H * V + i * G * N:H * V + (i + 1) * G * N].reshape(G, N)[pick] for i in (0, 1))
+            dt = np.logaddexp(0, x[s.x_dt:s.x_dt + H] + self._get(map_act, s.dt_bias, H))
+            g = np.exp(-np.exp(self._get(map_act, s.a_log, H)) * dt)
+            S = self._get(s.state_map, base + s.s_off, H * N * V).reshape(H, N, V) if p else np.zeros((H, N, V))
+            S = g[:, None, None] * S + dt[:, None, None] * B[:, :, None] * u[:, None, :]
+            self._put(s.state_map, base + s.s_off, S)
+            self._put(map_act, s.out + r * s.out_stride, np.einsum('hnv,hn->hv', S, C) + self._get(map_act, s.skip, H)[:, None] * u)
+
+    def experts_dev(self, map_act, map_opnd, map_wt, h, h_shared, rows):
+        s = self._spec(h, _MOE)
+        n, E = s.experts + s.identity, s.width
+        if s.shared_ff and rows > 1:
+            sh = self._spec(h_shared, _LINEAR)
+            self.linear_dev(map_act, map_opnd, map_wt, h_shared, 0, rows)
+        F16 = (s.ff + 15) // 16 * 16
+        for r in range(rows):
+            z = self._get(map_act, s.logits + r * s.logits_stride, n + (1 if s.shared_ff else 0))
+            sc = np.exp(z[:n] - z[:n].max())
+            sc = sc / sc.sum()
+            ids = np.argsort(-(sc + self._get(map_act, s.correction, n)), kind='stable')[:s.top]
+            h32 = self._get(map_act, s.x + r * s.x_stride, E)
+            x = self._get(map_opnd, s.opnd + r * s.k_stride, E) if rows > 1 else h32
+            y = np.zeros(E)
+            for j, e in enumerate(int(i) for i in ids):
+                if e >= s.experts:
+                    y += sc[e] * h32
+                    continue
+                gu = (self._get(map_wt, s.gate_up + e * s.gate_up_step, 2 * F16 * s.k_stride).reshape(-1, s.k_stride)[:, :E] @ x).reshape(-1, 2, 16)
+                a = (_silu(gu[:, 0]) * gu[:, 1]).reshape(-1)[:s.ff]
+                if rows > 1:
+                    o = s.act_opnd + (r * s.top + j) * s.ff_stride
+                    self._put(map_opnd, o, a)
+                    a = self._get(map_opnd, o, s.ff)
+                y += sc[e] * (self._get(map_wt, s.down + e * s.down_step, E * s.ff_stride).reshape(E, s.ff_stride)[:, :s.ff] @ a)
+            if s.shared_ff:
+                if rows > 1:
+                    v = self._get(map_act, sh.out + r * sh.out_stride, E)
+                else:
+                    W = self._get(map_wt, s.shared_down, E * s.shared_ff_stride).reshape(E, s.shared_ff_stride)[:, :s.shared_ff]
+                    v = W @ self._get(map_act, s.shared_act, s.shared_ff)
+                y += _sig(z[n]) * v
+            o = s.out + r * s.out_stride
+            self._put(map_act, o, y + (self._get(map_act, o, E) if s.epi else 0.0))
+
+    def embed_bigram_dev(self, map_act, map_src, h, locs, n_seq, rows, seq0, pos, post=False):
+        s = self._spec(h, _BIGRAM)
+        toks = self._get(map_act, 0, self.maps[map_act].n)[self.res[locs].view(np.uint32)[:n_seq * rows]].astype(np.int64)
+        for r, slot, p in self._tokens(n_seq, rows, seq0, pos):
+            at = slot * s.seq_stride + s.prev_off
+            pair = (int(self._get(s.state_map, at, 1)[0]) * s.mul_prev + int(toks[r]) * s.mul_cur) % s.buckets if p else s.buckets
+            self._put(s.state_map, at, [toks[r]])
+            self._put(map_act, s.dst + r * s.width, self._get(map_src, s.table + int(toks[r]) * s.width, s.width) * s.scale
+                      + self._get(map_src, s.pairs + pair * s.width, s.width))
