@@ -139,10 +139,7 @@ k_space_prep(const SSpec s, const float* __restrict__ act, const float* __restri
     const uint32_t t = tid & 15u;
     const bool in = c0 + t < m;
     const float d = in ? softplus_f(act[s.x + (uint64_t)(c0 + t) * s.x_stride + s.x_dt + h] + act[s.dt_bias + h]) : 0.f;
-    float l = -fminf(expf(act[s.a_log + h]) * d, NO_MEMORY) * 1.44269504f;
-#pragma unroll
-    for (int o = 1; o < 16; o <<= 1) { const float u = __shfl_up(l, o, 16); if ((int)t >= o) l += u; }
-    if (tid < CH) { dt[t] = d; lg[t] = l; }
+    if (tid < CH) { dt[t] = d; lg[t] = -fminf(expf(act[s.a_log + h]) * d, NO_MEMORY) * 1.44269504f; }
   }
   for (uint32_t i = tid; i < sd.Vp; i += 256u) {
     if (i < V) conv(h * V + i, [&](int t, float v) { oX[t * sd.Vp + i] = v; });
@@ -152,9 +149,15 @@ k_space_prep(const SSpec s, const float* __restrict__ act, const float* __restri
     }
   }
   __syncthreads();
+  // Decays between two tokens from the logarithms between them: the difference of two long sums would keep the rounding of
+  // everything ahead of both.
   const uint32_t t = tid >> 4, r = tid & 15u;
-  oM[t * 16u + r] = r <= t ? __builtin_amdgcn_exp2f(lg[t] - lg[r]) * dt[r] : 0.f;
-  if (tid < CH) { oE[tid] = __builtin_amdgcn_exp2f(lg[tid]); oG[tid] = __builtin_amdgcn_exp2f(lg[CH - 1u] - lg[tid]) * dt[tid]; }
+  float l = 0.f, e = 0.f;
+#pragma unroll
+  for (uint32_t i = 0; i < CH; i++) { l += i > r && i <= t ? lg[i] : 0.f; e += i <= r ? lg[i] : 0.f; }
+  l = r <= t ? __builtin_amdgcn_exp2f(l) * dt[r] : 0.f;
+  oM[t * 16u + r] = l;
+  if (t == CH - 1u) { oE[r] = __builtin_amdgcn_exp2f(e); oG[r] = l; }
 }
 
 // Four waves share the state rows (NT tiles of 16 each); a tile's accumulator holds rows 4 g + i of lane group g, which
