@@ -145,6 +145,25 @@ def mixer_config(width, ff, heads, head_dim, kv_heads, n_layer=4, n_vocab=32768,
     return MixerConfig(arch="Vomotar", n_vocab=n_vocab, n_embd=width, norm_groups=4, norm_eps=1e-6, layers=layers)
 
 
+def zaparax_config(width, ff, heads, head_dim, kv_heads, n_layer=4, n_vocab=32768, window=8192, experts=32, identity=2, top=6):
+    """A Zaparax model with the proportions of a real one: state-space and attention layers in turn, an inner width of twice
+    the model's in heads of 64 with 128 state rows, and a mixture whose chosen and shared experts are together `ff` wide (the
+    shared one as wide as two of the others)."""
+    from .feed_forward import Experts
+    from .mixers import StateSpace, WindowAttention
+    from .models import BigramTable, MixerConfig, MixerLayer
+    one = ff // (top + 2)
+    layers = []
+    for i in range(n_layer):
+        if i % 2 == 0:
+            m = StateSpace(2 * width // 64, 8, 128, 64, 4, 8)
+        else:
+            m = WindowAttention(heads, kv_heads, head_dim, head_dim, head_dim ** -0.5, window, 50.0, 0.1, 8192)
+        layers.append(MixerLayer(m, Experts(experts, identity, top, one, 2 * one)))
+    return MixerConfig(arch="Zaparax", n_vocab=n_vocab, n_embd=width, norm_eps=1e-6, layers=layers, emb_scale=1.0, norm_add=1.0,
+                       post_norm=True, pairs=BigramTable(16384, 8191, 3))
+
+
 def make_mixer_model(cfg, seed=0, rank=None):
     """dict name -> uint16 bfloat16 patterns, random.  Matrices are cut from one pool of normal numbers (what they hold
     does not change what a step costs)."""
@@ -152,15 +171,24 @@ def make_mixer_model(cfg, seed=0, rank=None):
     rng = np.random.default_rng(seed)
     pool = rng.standard_normal(1 << 24, dtype=np.float32)
     rank = rank or 128
+    scaled = {}                                    # bfloat16 pool per scale
+
+    def cut(k, at, shape):
+        if k not in scaled:
+            scaled[k] = f32_to_bf16(pool * np.float32(k))
+        p, size = scaled[k], int(np.prod(shape))
+        return np.resize(np.roll(p, -at), shape) if at + size > p.size else p[at:at + size].reshape(shape)
+
     out = {}
     for n, shape in cfg.tensors().items():
         shape = tuple(rank if d is None else d for d in shape)
-        size = int(np.prod(shape))
-        at = int(rng.integers(0, pool.size))
-        w = np.resize(np.roll(pool, -at) if size >= pool.size else np.concatenate([pool[at:at + size], pool[:max(0, at + size - pool.size)]]), shape)
+        at, last = int(rng.integers(0, pool.size)), n.split(".")[-1]
         if len(shape) == 1:
-            w = {"A_log": -2.0 + 0.5 * w, "dt_bias": -3.0 + 0.5 * w, "r1": 0.5 + 0.1 * w, "r2": 0.3 + 0.05 * w}.get(n.split(".")[-1], 1.0 + 0.1 * w)
-        elif not n.endswith(".conv") and n != "embed":
-            w = w * np.float32(shape[-1] ** -0.5)
-        out[n] = f32_to_bf16(np.asarray(w, np.float32))
+            centre, spread = {"A_log": (-2.0, 0.5), "dt_bias": (-3.0, 0.5), "r1": (0.5, 0.1), "r2": (0.3, 0.05), "sink": (0.0, 1.0), "b": (0.0, 0.1),
+                              "correction": (0.0, 0.01)}.get(last, (1.0, 0.1))
+            if "norm" in n and ".mix." not in n:
+                centre -= cfg.norm_add
+            out[n] = f32_to_bf16(np.float32(centre) + np.float32(spread) * pool[:shape[0]])
+        else:
+            out[n] = cut(1.0 if last == "conv" or n in ("embed", "bigram") else shape[-1] ** -0.5, at, shape)
     return out

@@ -417,57 +417,79 @@ MIXER_SIZES = {"2048": dict(width=2048, ff=8192, heads=16, head_dim=128, kv_head
                "4096": dict(width=4096, ff=14336, heads=32, head_dim=128, kv_heads=8)}
 
 
-def measure_mixers(gpu, A, synth, DecodeEngine, steps, warmup, n_prompt, sizes, chunk=None, only=None):
-    """Layered mixer model (Vomotar design, bfloat16 weights) beside the Llama shape (Q4_0 body, Q8_0 head) of equal
-    width, feed-forward, heads, depth and vocabulary: prefill of an n_prompt-token random prompt and bs = 1 greedy decoding
-    behind it, both with one step of lookahead.  Four layers; a step's bytes are the weights read once, the states
-    read and written and the visible keys and values; a prompt's work is two operations per weight and token."""
-    from adam_amd.engine import ModelConfig
+def mixer_step_bytes(cfg, params, pos):
+    """Bytes a decode step at position pos has to move: the weights it takes part in, states read and written, visible keys
+    and values (bfloat16).  Of a mixture the chosen and the shared experts count; identity experts at their share."""
+    att = 0
+    for L in cfg.layers:
+        m = getattr(L.mixer, "left", L.mixer)
+        seen = pos % m.chunk if hasattr(m, "chunk") else min(pos, m.window) if hasattr(m, "window") else 0
+        if seen:
+            att += 2 * m.kv_heads * (m.dim + m.vdim) * seen
+    return 2 * params + 8 * sum(L.mixer.state_size() for L in cfg.layers) + att
+
+
+def mixer_params(cfg, W):
+    """Matrix elements one token is multiplied by."""
+    params = sum(w.size for n, w in W.items() if w.ndim == 2 and n not in ("embed", "bigram") and not n.endswith(".conv"))
+    for L in cfg.layers:
+        if hasattr(L.ff, "experts"):
+            f = L.ff
+            params -= 3 * f.ff * cfg.n_embd * (f.experts - f.top * f.experts / (f.experts + f.identity))
+    return params
+
+
+def measure_mixer_engine(gpu, A, cfg, W, steps, warmup, n_prompt, chunk):
     from adam_amd.mixer_engine import MixerEngine
+    eng = MixerEngine(gpu, cfg, W, A=A, prefill_chunk=chunk)
+    prompt = [int(t) for t in np.random.default_rng(0).integers(0, cfg.n_vocab, n_prompt)]
+    eng.prefill(prompt)                                         # warm-up: allocations, code objects
+    eng.reset()
+    gpu.sync()
+    t0 = time.perf_counter()
+    eng.prefill(prompt)
+    gpu.sync()
+    pre = time.perf_counter() - t0
+    pos, runs = n_prompt, []
+
+    def run(n):
+        nonlocal pos
+        for _ in range(n):
+            eng._forward(None, pos, from_device=True)
+            eng._wait_tokens(eng._feed_ticket)
+            pos += 1
+    run(warmup)
+    for _ in range(3):
+        gpu.sync()
+        gpu.reset_native_stats()
+        t0 = time.perf_counter()
+        run(steps)
+        gpu.sync()
+        runs.append(time.perf_counter() - t0)
+    launches = gpu.get_native_stats()["dispatch_count"] / steps
+    params = mixer_params(cfg, W)
+    step_bytes, dt = mixer_step_bytes(cfg, params, pos), sorted(runs)[1] / steps
+    return {"prefill_tok/s": round(n_prompt / pre, 1), "prefill_TFLOP/s": round(2e-12 * params * n_prompt / pre, 1),
+            "decode_tok/s": round(1 / dt, 1), "ms_per_step": round(1e3 * dt, 4), "step_MB": round(step_bytes / 1e6, 1),
+            "frac_of_hbm_peak": round(step_bytes / dt / 1e9 / HBM_PEAK_GBPS, 4), "launches_per_token": round(launches, 1)}
+
+
+def measure_mixers(gpu, A, synth, DecodeEngine, steps, warmup, n_prompt, sizes, chunk=None, only=None):
+    """Layered mixer models (bfloat16 weights), Vomotar and Zaparax designs, beside the Llama shape (Q4_0 body, Q8_0 head) of
+    equal width, feed-forward (a mixture: what a token takes of it), heads, depth and vocabulary: prefill of an n_prompt-token
+    random prompt and bs = 1 greedy decoding behind it, with one step of lookahead.  Four layers; a prompt's work is two
+    operations per weight and token.  `only`: the legs to run."""
+    from adam_amd.engine import ModelConfig
     out = {}
     for name in sizes:
         sz = MIXER_SIZES[name]
         row = {}
-        if only in (None, "mixer"):
-            cfg = synth.mixer_config(**sz)
-            W = synth.make_mixer_model(cfg)
-            eng = MixerEngine(gpu, cfg, W, A=A, prefill_chunk=chunk or 2048)
-            prompt = [int(t) for t in np.random.default_rng(0).integers(0, cfg.n_vocab, n_prompt)]
-            eng.prefill(prompt)                                         # warm-up: allocations, code objects
-            eng.reset()
-            gpu.sync()
-            t0 = time.perf_counter()
-            eng.prefill(prompt)
-            gpu.sync()
-            pre = time.perf_counter() - t0
-            pos, runs = n_prompt, []
-
-            def run(n):
-                nonlocal pos
-                for _ in range(n):
-                    eng._forward(None, pos, from_device=True)
-                    eng._wait_tokens(eng._feed_ticket)
-                    pos += 1
-            run(warmup)
-            for _ in range(3):
-                gpu.sync()
-                gpu.reset_native_stats()
-                t0 = time.perf_counter()
-                run(steps)
-                gpu.sync()
-                runs.append(time.perf_counter() - t0)
-            launches = gpu.get_native_stats()["dispatch_count"] / steps
-            params = sum(w.size for n, w in W.items() if w.ndim == 2 and n != "embed" and not n.endswith(".conv"))
-            att = sum(2 * L.mixer.left.kv_heads * (L.mixer.left.dim + L.mixer.left.vdim) * (pos % L.mixer.left.chunk)
-                      for L in cfg.layers if hasattr(L.mixer, "left"))
-            step_bytes = 2 * params + 8 * sum(L.mixer.state_size() for L in cfg.layers) + att
-            dt = sorted(runs)[1] / steps
-            row["mixer"] = {"prefill_tok/s": round(n_prompt / pre, 1), "prefill_TFLOP/s": round(2e-12 * params * n_prompt / pre, 1),
-                            "decode_tok/s": round(1 / dt, 1), "ms_per_step": round(1e3 * dt, 4), "step_MB": round(step_bytes / 1e6, 1),
-                            "frac_of_hbm_peak": round(step_bytes / dt / 1e9 / HBM_PEAK_GBPS, 4), "launches_per_token": round(launches, 1)}
-            log(f"mixer {name}: {row['mixer']}")
-            del eng, W
-        if only in (None, "llama"):
+        for leg, make in (("mixer", synth.mixer_config), ("zaparax", synth.zaparax_config)):
+            if leg in only:
+                cfg = make(**sz)
+                row[leg] = measure_mixer_engine(gpu, A, cfg, synth.make_mixer_model(cfg), steps, warmup, n_prompt, chunk or 2048)
+                log(f"{leg} {name}: {row[leg]}")
+        if "llama" in only:
             cfg = ModelConfig(arch="llama", n_vocab=32768, n_embd=sz["width"], n_head=sz["heads"], n_head_kv=sz["kv_heads"], n_layer=4,
                               n_ff=sz["ff"], head_dim=128, head_dim_kv=128, norm_eps=1e-5, rope_base_global=5e5, rope_base_local=5e5)
             t = synth.make_model(cfg, seed=0, sigma=0.02)
@@ -500,7 +522,7 @@ def main():
                          "loop either way")
     ap.add_argument("--batch", type=int, default=16, help="sequences decoded in lockstep (config 5 leg, --only batch)")
     ap.add_argument("--only", default=None, choices=["roofline", "gemv", "probe", "attention", "gemm", "prefill", "batch", "mixers", "mixers-mixer",
-                                                         "mixers-llama"],
+                                                         "mixers-llama", "zaparax", "mixers-zaparax"],
                     help="roofline: just the 28672x4096 GEMV (one kernel row in a rocprofv3 --stats table); "
                          "gemv: that shape, 4096x4096 and 4096x14336; probe: plain read/copy kernels of known "
                          "size (reference points for rocprofv3 --pmc FETCH_SIZE / WRITE_SIZE); attention: GQA "
@@ -510,7 +532,7 @@ def main():
                          "layer); batch: --batch random prompts of --prompt (default 1024) tokens prefilled in "
                          "chunks of 512, then --steps lockstep decode steps of --workload; mixers: the layered mixer model "
                          "beside the Llama shape of equal size, at two sizes (mixers-mixer / mixers-llama: one of the "
-                         "two)")
+                         "two); zaparax: the Zaparax model beside the layered mixer model of equal size (mixers-zaparax: the first alone)")
     ap.add_argument("--mixer-size", default=None, choices=list(MIXER_SIZES), help="--only mixers: one width alone")
     ap.add_argument("--skip-reference", action="store_true",
                     help="--only prefill: time the chunked prompt alone (chunks of --prefill-chunk, default the whole "
@@ -531,11 +553,11 @@ def main():
             args.steps = 128
         print(json.dumps(measure_model_batched(args, A, synth, DecodeEngine)), flush=True)
         return
-    if args.only and args.only.startswith("mixers"):
+    if args.only and (args.only.startswith("mixers") or args.only == "zaparax"):
         gpu = A.init()
-        one = args.only.partition("-")[2] or None
+        legs = {"mixers": ("mixer", "llama"), "zaparax": ("mixer", "zaparax")}.get(args.only) or (args.only.partition("-")[2],)
         print(json.dumps({"mixers": measure_mixers(gpu, A, synth, DecodeEngine, min(args.steps, 64), args.warmup, args.prompt or 4032,
-                                                   [args.mixer_size] if args.mixer_size else list(MIXER_SIZES), args.prefill_chunk, one)}), flush=True)
+                                                   [args.mixer_size] if args.mixer_size else list(MIXER_SIZES), args.prefill_chunk, legs)}), flush=True)
         gpu.shutdown()
         return
     if args.only:
