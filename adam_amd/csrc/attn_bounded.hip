@@ -608,8 +608,9 @@ static int run_portion(const ASpec& s, float* act, T* cache, uint32_t m, uint32_
 template <class T, bool WIN, int NC, int RG, int KI>
 static int run_step_as(const ASpec& s, float* act, T* cache, uint32_t n_seq, uint32_t seq0, uint32_t pos) {
   const uint32_t parts = cdiv(s.heads / s.kv_heads, RG), n = WIN ? std::min(pos + 1u, s.size) : pos % s.size + 1u, unit = STEP_WAVES * 4u * KI;
-  const uint32_t most = std::min<uint32_t>(MAX_SPANS, std::max<uint32_t>(1u, 2u * (uint32_t)g.n_cu / (s.kv_heads * parts * n_seq)));
-  const uint32_t span = cdiv(cdiv(n, std::min(most, cdiv(n, unit))), unit) * unit, spans = cdiv(n, span);
+  // no more workgroups than compute units: a few too many would take as long as twice as many
+  const uint32_t most = std::min<uint32_t>(MAX_SPANS, std::max<uint32_t>(1u, (uint32_t)g.n_cu / (s.kv_heads * parts * n_seq)));
+  const uint32_t span = std::max<uint32_t>(unit, cdiv(cdiv(n, most), 4u * KI) * 4u * KI), spans = cdiv(n, span);
   if (s.size > unit)      // at its full size from the first step on: a graph may be recording when the second span begins
     if (int r = scratch_need(g_parts, (size_t)n_seq * s.heads * MAX_SPANS * (s.vdim + 2) * 4)) return r;
   k_attn_step<T, WIN, NC, RG, KI><<<dim3(s.kv_heads * parts, spans, n_seq), STEP_WAVES * 64, 0, g.stream>>>(s, act, cache, (float*)g_parts.p, seq0, pos, span, parts);

@@ -68,20 +68,22 @@ k_embed_tokens(float* act, uint64_t act_elems, const uint8_t* __restrict__ src, 
   act[dst0 + i] = v;
 }
 
-// One workgroup per row: scale * row of the token table + row of the bigram table (AdamahBigramSpec).  The workgroup that
-// starts a sequence's rows is the only one to touch its previous token in the state map: it reads it and then leaves the
-// last row's token there.
+// One workgroup per row (and one that posts the tokens, if there is mail): scale * row of the token table + row of the
+// bigram table (AdamahBigramSpec).  The workgroup that starts a sequence's rows is the only one to touch its previous token
+// in the state map: it reads it and then leaves the last row's token there.
 template <bool BF>
 __global__ void __launch_bounds__(512)
 k_embed_bigram(const AdamahBigramSpec s, float* act, uint64_t act_elems, const uint8_t* __restrict__ src, const uint32_t* __restrict__ tok_locs,
                float* state, uint32_t rows, uint32_t seq0, uint32_t pos, TokenMail* mail, uint32_t ticket, uint32_t n_tok) {
-  if (mail && blockIdx.x == 0 && threadIdx.x < 64u) {
+  if (mail && blockIdx.x + 1u == gridDim.x) {                               // a workgroup of its own, behind the rows
+    if (threadIdx.x >= 64u) return;
     if (threadIdx.x < n_tok) mail->val[threadIdx.x] = tok_locs[threadIdx.x] < act_elems ? act[tok_locs[threadIdx.x]] : 0.0f;
     __threadfence_system();
     if (threadIdx.x == 0) {
       mail->n = n_tok;
       __hip_atomic_store(&mail->ticket, ticket, __ATOMIC_RELEASE, __HIP_MEMORY_SCOPE_SYSTEM);
     }
+    return;
   }
   const uint32_t r = blockIdx.x, seq = r / rows, t = r - seq * rows;       // rows tokens of each sequence
   float* kept = state + (uint64_t)(seq0 + seq) * s.seq_stride + s.prev_off;
@@ -91,6 +93,7 @@ k_embed_bigram(const AdamahBigramSpec s, float* act, uint64_t act_elems, const u
   const uint64_t tok = ok ? (uint32_t)tf : 0u, prev = ok ? (uint32_t)pf : 0u;
   const uint64_t pair = pos + t == 0u ? s.buckets : (prev * s.mul_prev + tok * s.mul_cur) % s.buckets;
   const uint64_t a = s.table + tok * s.width, b = s.pairs + pair * s.width;
+#pragma unroll 8
   for (uint32_t i = threadIdx.x; i < s.width; i += 512u) {
     float v = 0.0f;
     if (ok) v = BF ? fmaf(__uint_as_float((uint32_t)((const uint16_t*)src)[a + i] << 16), s.scale, __uint_as_float((uint32_t)((const uint16_t*)src)[b + i] << 16))
@@ -219,7 +222,8 @@ int adamah_hip_embed_bigram_dev(uint32_t map_act, uint32_t map_src, uint32_t h_s
     *ticket_out = ticket;
     mail = g_mail_dev + ticket % MAIL_SLOTS;
   }
-#define EMBED(BF) k_embed_bigram<BF><<<(uint32_t)m, 512, 0, g.stream>>>(*s, (float*)ma->buf, ma->n_elems, ms->buf, tl, (float*)mt->buf, rows, seq0,                                                                       pos, mail, ticket, (uint32_t)m)
+#define EMBED(BF) k_embed_bigram<BF><<<(uint32_t)m + (mail ? 1u : 0u), 512, 0, g.stream>>>(*s, (float*)ma->buf, ma->n_elems, ms->buf, tl, \
+                                                                             (float*)mt->buf, rows, seq0, pos, mail, ticket, (uint32_t)m)
   if (ms->dtype == DTYPE_BF16) EMBED(true); else EMBED(false);
 #undef EMBED
   count_launch();
