@@ -235,17 +235,18 @@ def test_window_attention_with_parts_left_out(hip, dtype, kw):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_window_attention_over_several_spans_of_keys(hip, dtype):
-    """A window of 1500 tokens: a decoded token reads its keys in spans, the ring turns over inside one of them."""
-    note(f"window attention, wide window {dtype}")
-    R = 1500
-    run, _, _ = window_pair(hip, 4, 2, 32, 40, R, dtype, 300, 1, seed=5, scale=0.6, slope=0.003)
+@pytest.mark.parametrize("H,G,D,V,R,total,ones", [(4, 2, 32, 40, 1500, 1900, (300, 1200, 1502)), (64, 64, 8, 8, 700, 950, (300, 601))])
+def test_window_attention_over_several_spans_of_keys(hip, H, G, D, V, R, total, ones, dtype):
+    """A wide window: a decoded token reads its keys in spans, the ring turns over inside one of them; with many key heads the
+    spans grow past what a workgroup takes at once."""
+    note(f"window attention, wide window, H {H} {dtype}")
+    run, _, _ = window_pair(hip, H, G, D, V, R, dtype, 300, 1, seed=5, scale=0.6, slope=0.003)
     pos = 0
-    while pos < 1900:
-        m = min(300, 1900 - pos)
+    while pos < total:
+        m = min(300, total - pos)
         run(1, m, 0, pos)
         pos += m
-        if pos in (300, 1200, 1502):
+        if pos in ones:
             run(1, 1, 0, pos)
             pos += 1
     for pos in range(pos, pos + 4):
