@@ -10,7 +10,7 @@ zeros), 2 operand rows of multi-row products, 3 float32 recurrent state, 14 key-
 `dtype='bfloat16'`: operand rows and cache in bfloat16.  'float32': both in float32 and every product in float32; the
 weights are stored in bfloat16 either way, which is exact for a model file that holds them so.
 
-What a sequence keeps is bounded: recurrent state, convolution inputs and one attention chunk per layer, so there is
+What a sequence keeps is bounded: recurrent state, convolution inputs and one attention chunk or window per layer, so there is
 no cache length to choose and no end to a sequence (positions count up to 2^24, where float32 angles stop being exact).
 """
 import numpy as np
